@@ -131,6 +131,8 @@ class ModelPresets:
         "fusasun-1b": "fusasun-1b",
         "lumedra-tiny": "lumedra-tiny",
         "lumedra-1b": "lumedra-1b",
+        "kafilorn-tiny": "kafilorn-tiny",
+        "kafilorn-1b": "kafilorn-1b",
     })
     embedders: dict = field(default_factory=lambda: {
         "nomic-embed-text": "nomic-embed-text",

@@ -8,10 +8,11 @@ import torch
 
 from ..parallel.tp import SINGLE, TPGroup
 from .bert import EncoderModel
-from .configs import (DECODERS, ENCODERS, DecoderConfig, EncoderConfig, FusasunConfig, LebepelConfig, LumedraConfig, PemidraConfig, decoder_config,
+from .configs import (DECODERS, ENCODERS, DecoderConfig, EncoderConfig, FusasunConfig, KafilornConfig, LebepelConfig, LumedraConfig, PemidraConfig, decoder_config,
                       encoder_config)
 from . import llama
 from .fusasun import FusasunModel
+from .kafilorn import KafilornModel
 from .lebepel import LebepelModel
 from .llama import LlamaModel
 from .lumedra import LumedraModel
@@ -20,10 +21,11 @@ from .pemidra import PemidraModel, ranks_from_state_dict
 
 # decoder architectures by ``cfg.arch``
 DECODER_CLASSES = {"llama": LlamaModel, "opt": OPTModel, "lebepel": LebepelModel, "pemidra": PemidraModel,
-                   "fusasun": FusasunModel, "lumedra": LumedraModel}
+                   "fusasun": FusasunModel, "lumedra": LumedraModel, "kafilorn": KafilornModel}
 # designs with a checkpoint format of their own (config.json read by ``<Config>.from_json``, tensors by
 # ``load_state_dict_native``)
-NATIVE_CONFIGS = {"lebepel": LebepelConfig, "pemidra": PemidraConfig, "fusasun": FusasunConfig, "lumedra": LumedraConfig}
+NATIVE_CONFIGS = {"lebepel": LebepelConfig, "pemidra": PemidraConfig, "fusasun": FusasunConfig, "lumedra": LumedraConfig,
+                  "kafilorn": KafilornConfig}
 
 
 def _load_safetensors_dir(path: str) -> dict:
@@ -120,5 +122,6 @@ def build_encoder(name: str | EncoderConfig, device="cpu", dtype=torch.bfloat16,
 
 
 __all__ = ["build_decoder", "build_encoder", "load_decoder_dir", "checkpoint_architecture", "DECODER_CLASSES",
-           "LebepelConfig", "LebepelModel", "PemidraConfig", "PemidraModel", "FusasunConfig", "FusasunModel", "LumedraConfig", "LumedraModel", "NATIVE_CONFIGS", "DECODERS", "ENCODERS", "DecoderConfig", "EncoderConfig",
+           "LebepelConfig", "LebepelModel", "PemidraConfig", "PemidraModel", "FusasunConfig", "FusasunModel", "LumedraConfig", "LumedraModel",
+           "KafilornConfig", "KafilornModel", "NATIVE_CONFIGS", "DECODERS", "ENCODERS", "DecoderConfig", "EncoderConfig",
            "LlamaModel", "OPTModel", "EncoderModel"]

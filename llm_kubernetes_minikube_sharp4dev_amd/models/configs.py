@@ -280,6 +280,98 @@ class LumedraConfig:
                            for l in self.layers]}
 
 
+@dataclass
+class KafilornConfig:
+    """The Kafilorn design: a residual stream kept as ``streams`` mixed copies (every sublayer reads one learned combination of
+    them, layer-normed, and its result is written back while the copies are mixed with each other), two mixers in any
+    order -- ``mlstm`` (a matrix memory with exponential gates) and ``latent_attention`` (sliding window with a learned sink
+    over a cached latent, which later layers may share: mixer ``kv_from``) -- and a feed-forward that is dense (squared
+    relu), a mixture of experts (softmax router with a choice correction and group-limited choice, a shared expert) or
+    absent.  Scaled embedding, own LM head with a logit scale.  Every size and constant comes from the checkpoint's
+    ``config.json`` (:meth:`from_json`)."""
+    name: str
+    vocab_size: int
+    hidden: int
+    layers: list                 # [HybridLayer]
+    streams: int = 1
+    norm_eps: float = 1e-6
+    embed_scale: float = 1.0
+    logit_scale: float = 1.0
+    max_position: int = 1 << 20  # nothing in the design bounds a sequence; engines pass their own limit
+    arch: str = "kafilorn"
+    bos_token_id: int = 0
+    eos_token_ids: tuple = ()
+    tie_word_embeddings: bool = False
+
+    MIXERS = ("mlstm", "latent_attention")
+    MLPS = ("dense", "moe")
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    def __post_init__(self):
+        for i, l in enumerate(self.layers):
+            if l.type not in self.MIXERS:
+                raise ValueError(f"unknown mixer type {l.type!r}")
+            if l.mlp is not None and l.mlp.get("kind") not in self.MLPS:
+                raise ValueError(f"unknown feed-forward kind {l.mlp.get('kind')!r}")
+            j = l.mixer.get("kv_from") if l.type == "latent_attention" else None
+            if j is None:
+                continue
+            if not 0 <= j < i or self.layers[j].type != "latent_attention" or self.layers[j].mixer.get("kv_from") is not None:
+                raise ValueError(f"layer {i}: kv_from {j} must name an earlier latent attention layer with a cache of its own")
+            a, b = l.mixer, self.layers[j].mixer
+            if (a["kv_rank"], a["rot_dim"]) != (b["kv_rank"], b["rot_dim"]):
+                raise ValueError(f"layers {i} and {j} share a latent of different sizes")
+        if self.streams < 1:
+            raise ValueError("at least one stream")
+
+    @classmethod
+    def from_json(cls, d: dict, name: str = "kafilorn") -> "KafilornConfig":
+        layers = [HybridLayer(l["type"], dict(l["mixer"]), dict(l["mlp"]) if l.get("mlp") else None)
+                  for l in d["layers"]]
+        return cls(name=name, vocab_size=int(d["vocab"]), hidden=int(d["width"]), layers=layers, streams=int(d.get("streams", 1)),
+                   norm_eps=float((d.get("norm") or {}).get("eps", 1e-6)),
+                   embed_scale=float((d.get("embedding") or {}).get("scale", 1.0)), logit_scale=float(d.get("logit_scale", 1.0)),
+                   max_position=int(d.get("max_positions", 1 << 20)))
+
+    def to_json(self) -> dict:
+        return {"architecture": "Kafilorn", "vocab": self.vocab_size, "width": self.hidden, "norm": {"eps": self.norm_eps},
+                "streams": self.streams, "embedding": {"scale": self.embed_scale}, "logit_scale": self.logit_scale,
+                "layers": [{"type": l.type, "mixer": dict(l.mixer), "mlp": dict(l.mlp) if l.mlp else None}
+                           for l in self.layers]}
+
+
+def kafilorn_layers(n: int, heads: int, head_dim: int, dense_ff: int, expert_ff: int = 0, experts: int = 0, top: int = 2,
+                    window: int = 1024, rot_dim: int = 64, q_rank: int = 768, kv_rank: int = 512, groups: int = 4, keep: int = 2,
+                    shared_ff: int = 0, gate_cap: float = 15.0, pattern=("mlstm", "latent_attention", "shared_latent")) -> list:
+    """``n`` layers cycling through ``pattern`` with one set of head sizes (presets and benchmarks); ``shared_latent``: latent
+    attention over the latest latent that a layer caches.  Every second layer has experts, the others a dense feed-forward
+    (``experts`` 0: all dense)."""
+    out, last = [], None
+    for i in range(n):
+        t = pattern[i % len(pattern)]
+        if t == "mlstm":
+            mixer = {"heads": heads, "dim": head_dim, "vdim": head_dim, "gate_cap": gate_cap}
+        else:
+            mixer = {"heads": heads, "dim": head_dim, "rot_dim": rot_dim, "vdim": head_dim, "q_rank": q_rank, "kv_rank": kv_rank,
+                     "scale": (head_dim + rot_dim) ** -0.5, "rot": {"base": 10000.0, "dims": rot_dim}, "mask": {"size": window}}
+            if t == "shared_latent" and last is not None:
+                mixer["kv_from"] = last
+            else:
+                last = i
+        if experts and i % 2 == 1:
+            mlp = {"kind": "moe", "expert": {"ff": expert_ff},
+                   "router": {"experts": experts, "top": top, "groups": {"count": groups, "keep": keep}}}
+            if shared_ff:
+                mlp["shared"] = {"ff": shared_ff}
+        else:
+            mlp = {"kind": "dense", "ff": dense_ff}
+        out.append(HybridLayer("mlstm" if t == "mlstm" else "latent_attention", mixer, mlp))
+    return out
+
+
 def lumedra_layers(n: int, heads: int, head_dim: int, ff: int, experts: int = 0, top: int = 2, kv_heads: Optional[int] = None,
                    window: int = 1024, keep_first: int = 4, softcap: float = 30.0, rot_dim: int = 64, q_rank: int = 768,
                    kv_rank: int = 512, groups: int = 4, keep: int = 2, shared_ff: int = 0, router_scale: float = 2.5,
@@ -431,6 +523,16 @@ DECODERS.update({
     "lumedra-1b": LumedraConfig("lumedra-1b", 32768, 2048, lumedra_layers(18, 16, 128, 704, 16, 4, kv_heads=4, shared_ff=1408)),
 })
 
+DECODERS.update({
+    # several mixed residual streams, matrix-memory and shared-latent attention layers (random-init presets)
+    "kafilorn-tiny": KafilornConfig("kafilorn-tiny", 32768, 128, kafilorn_layers(4, 4, 24, 80, 24, 6, 2, window=20, rot_dim=8, q_rank=48,
+                                                                                  kv_rank=40, groups=3, keep=2, shared_ff=40,
+                                                                                  gate_cap=8.0), streams=3, embed_scale=2.0,
+                                    logit_scale=0.5),
+    "kafilorn-1b": KafilornConfig("kafilorn-1b", 32768, 2048, kafilorn_layers(18, 16, 128, 8192, 704, 16, 4, kv_rank=512, q_rank=1024,
+                                                                              shared_ff=1408), streams=4),
+})
+
 ENCODERS = {
     "bge-base": EncoderConfig("bge-base", "bert", 12, 768, 12, 3072, 30522, pooling="cls"),
     "minilm-l6": EncoderConfig("minilm-l6", "bert", 6, 384, 12, 1536, 30522, pooling="mean"),
@@ -458,6 +560,29 @@ def encoder_config(name: str, **overrides) -> EncoderConfig:
 
 
 def param_count(cfg) -> int:
+    if isinstance(cfg, KafilornConfig):
+        W, S = cfg.hidden, cfg.streams
+        n = 2 * cfg.vocab_size * W + W
+        for l in cfg.layers:
+            m = l.mixer
+            if l.type == "mlstm":
+                n += W * m["heads"] * (2 * m["dim"] + 3 * m["vdim"] + 2) + m["heads"] * (m["vdim"] + 2)
+            else:
+                qd = m["dim"] + m["rot_dim"]
+                n += m["q_rank"] * (W + 1 + m["heads"] * qd) + m["kv_rank"] * m["heads"] * (m["dim"] + m["vdim"]) \
+                    + W * m["heads"] * m["vdim"] + m["heads"]
+                if m.get("kv_from") is None:
+                    n += W * (m["kv_rank"] + m["rot_dim"]) + m["kv_rank"]
+            n += W + 2 * S + S * S
+            if l.mlp:
+                n += W + 2 * S + S * S
+            if l.mlp and l.mlp["kind"] == "dense":
+                n += 2 * W * l.mlp["ff"]
+            elif l.mlp:
+                r = l.mlp["router"]
+                n += r["experts"] * (3 * W * l.mlp["expert"]["ff"] + W + 1)
+                n += 3 * W * l.mlp["shared"]["ff"] if l.mlp.get("shared") else 0
+        return n
     if isinstance(cfg, LumedraConfig):
         W, n = cfg.hidden, cfg.vocab_size * cfg.hidden + cfg.hidden
         for l in cfg.layers:

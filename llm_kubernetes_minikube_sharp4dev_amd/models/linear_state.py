@@ -1,6 +1,7 @@
-"""Linear-state mixers over the engine's per-sequence state slots: retention, lightning attention (retention on
+"""Linear-state mixers over the engine's per-sequence state slots: the matrix memory with exponential gates
+(``mlstm_mixer``, a recurrence of its own: ``ops.mlstm``), retention, lightning attention (retention on
 activated projections with one norm over all heads), the gated delta rule (with short causal convolutions on
-q, k, v) and the generalized delta rule.  All are members of
+q, k, v) and the generalized delta rule.  All but the first are members of
 
     S_t = diag(w_t) S_(t-1) - p_t (z_t^T S_(t-1)) + k_t v_t^T,    o_t = S_t^T q_t
 
@@ -123,6 +124,47 @@ def lightning_mixer(h, w_in, rows: FusedRows, decay, norm_w, w_out, spec: Lightn
                        max_len=meta.max_seq_len, act=True)
     g = ops.head_norm_gate(o, rows.cols(u, "g"), norm_w, 1, eps, ops.GATE_SIGMOID, out_dtype)
     return ops.linear(g, w_out)
+
+
+@dataclass
+class MLSTMSpec:
+    """Matrix memory with exponential gates: per head log gates ``i = cap tanh(z_i / cap)`` and ``f = log sigmoid(cap tanh(z_f /
+    cap))`` (z: projections with bias, f32), ``S <- exp(f) S + exp(i) k v^T`` and a normaliser ``n <- exp(f) n + exp(i) k``, both relative
+    to a running maximum (``ops.mlstm``); output per head ``S^T q / max(|n.q|, 1 at the same scale)``, divided by its RMS,
+    times a weight, times ``sigmoid(W_g h)``, projected."""
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float = 15.0
+
+    @classmethod
+    def from_dict(cls, m: dict) -> "MLSTMSpec":
+        s = cls(int(m["heads"]), int(m["dim"]), int(m.get("vdim", m["dim"])), float(m["gate_cap"]))
+        if not ops.mlstm_supported(s.dim, s.vdim) or s.gate_cap <= 0:
+            raise ValueError(f"unsupported matrix-memory sizes {m}")
+        return s
+
+    def rows(self, width: int) -> FusedRows:
+        return FusedRows([("q", self.heads * self.dim), ("k", self.heads * self.dim), ("v", self.heads * self.vdim),
+                          ("g", self.heads * self.vdim)], fused_mult(width))
+
+    def make_state(self, slots: int, dtype, device):
+        return ops.mlstm_state(slots, self.heads, self.dim, self.vdim, device)
+
+    def state_bytes(self, dtype) -> int:
+        return sum(t.numel() * t.element_size() for t in ops.mlstm_state(1, self.heads, self.dim, self.vdim, "cpu"))
+
+
+def mlstm_mixer(h, w_in, w_gates, gate_bias, rows: FusedRows, norm_w, w_out, spec: MLSTMSpec, eps: float, state, meta, out_dtype):
+    """h [T, W] -> [T, W]: q | k | v | g in one projection, the gates in f32 beside it (``w_gates`` [2 heads, W]: input gate
+    rows, then forget gate rows), the recurrence (q scaled by dim^-1/2, f32 state), per-head unit RMS times a weight times
+    sigmoid(g), output projection."""
+    u = ops.linear(h, w_in)
+    gates = ops.gate_proj(h, w_gates, gate_bias, spec.heads, spec.gate_cap)
+    o = ops.mlstm_scan(rows.cols(u, "q"), rows.cols(u, "k"), rows.cols(u, "v"), gates, state, meta.seq_cu, meta.state_slots,
+                       meta.positions, spec.heads, spec.dim, spec.vdim, q_scale=spec.dim ** -0.5, max_len=meta.max_seq_len)
+    y = ops.head_norm_gate(o, rows.cols(u, "g"), norm_w, spec.heads, eps, ops.GATE_SIGMOID, out_dtype)
+    return ops.linear(y, w_out)
 
 
 @dataclass
