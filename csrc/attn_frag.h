@@ -1,6 +1,7 @@
 // Fragment helpers shared by the attention kernels that read a paged K cache [blocks, G, BS, dim] and a
 // key-contiguous V cache [blocks, G, vdim, BS] straight into MFMA operands (attn_sigmoid.hip,
-// attn_sink.hip): element traits of the two activation types and the S^T += K . Q^T step.
+// attn_sink.hip), and by the products that read rows straight from memory (moe.hip, head_linear.hip, row_proj.hip):
+// element traits of the two activation types, the S^T += K . Q^T step, a padded 16-byte fragment of a row.
 #pragma once
 #include "common.h"
 
@@ -34,6 +35,17 @@ LK_DEVICE floatx4 mma_qk(uint4_t a, uint4_t b, floatx4 c) {
     for (int e = 0; e < 4; ++e) c = __builtin_amdgcn_mfma_f32_16x16x4f32(fa[e], fb[e], c, 0, 0, 0);
     return c;
   }
+}
+
+// 16 bytes of row `r` at element k (EV elements; zeros past K): one vector load when the row allows it
+template <typename T>
+LK_DEVICE uint4_t frag(const T* r, int k, int K, bool vec) {
+  constexpr int EV = El<T>::V;
+  if (vec && k + EV <= K) return ld16(r + k);
+  alignas(16) T tmp[EV];
+#pragma unroll
+  for (int e = 0; e < EV; ++e) tmp[e] = k + e < K ? r[k + e] : T(0);
+  return *reinterpret_cast<const uint4_t*>(tmp);
 }
 
 }  // namespace

@@ -1746,6 +1746,186 @@ at::Tensor moe_gemm(const at::Tensor& x, const at::Tensor& order, const at::Tens
   return out;
 }
 
+// ---------------------------------------------------------------------------------------------
+// mixed residual streams, skinny f32 projections, matrix memory, attention over a cached latent
+std::vector<c10::optional<at::Tensor>> stream_hyper_norm(at::Tensor& x, int64_t S, const c10::optional<at::Tensor>& a,
+                                                         const c10::optional<at::Tensor>& b, const c10::optional<at::Tensor>& y,
+                                                         const c10::optional<at::Tensor>& yw, const c10::optional<at::Tensor>& mix,
+                                                         const c10::optional<at::Tensor>& wout, const c10::optional<at::Tensor>& win,
+                                                         const c10::optional<at::Tensor>& w, double eps, at::ScalarType out_dtype,
+                                                         const c10::optional<at::Tensor>& idx, double oscale) {
+  CHECK_CUDA(x); CHECK_F32(x); CHECK_CONTIG(x);
+  TORCH_CHECK(out_dtype == at::kBFloat16 || out_dtype == at::kFloat, "out dtype");
+  TORCH_CHECK(S >= 1 && S <= 8 && (x.dim() == 2 || (x.dim() == 3 && x.size(1) == S)), "x must be [T, S, W] or, while all copies are equal, [T, W]");
+  const long T = x.size(0);
+  const int W = x.size(-1), esz = out_dtype == at::kFloat ? 4 : 2;
+  auto rows_of = [&](const c10::optional<at::Tensor>& t, long rows, const char* what, long* stride) -> const void* {
+    if (!t) return nullptr;
+    CHECK_CUDA(*t); CHECK_LASTDIM(*t);
+    TORCH_CHECK(t->dim() == 2 && t->size(0) == rows && t->size(1) == W, what, " must be [", rows, ", ", W, "]");
+    TORCH_CHECK(t->scalar_type() == out_dtype, what, ": dtype must be the activations'");
+    *stride = t->stride(0);
+    return t->data_ptr();
+  };
+  long as = 0, bs = 0, ys = 0;
+  const void* ap = rows_of(a, T, "a", &as);
+  const void* bp_ = rows_of(b, T, "b", &bs);
+  int top = 0;
+  const float* ywp = nullptr;
+  if (y) {
+    TORCH_CHECK(yw.has_value(), "expert rows need their weights");
+    CHECK_CUDA(*yw); CHECK_F32(*yw); CHECK_CONTIG(*yw);
+    TORCH_CHECK(yw->dim() == 2 && yw->size(0) == T && yw->size(1) >= 1, "weights must be f32 [T, top]");
+    top = yw->size(1);
+    ywp = yw->data_ptr<float>();
+  }
+  const void* yp = rows_of(y, T * std::max(top, 1), "y", &ys);
+  const bool upd = ap || bp_ || yp;
+  TORCH_CHECK(upd || w.has_value(), "neither an update nor a norm");
+  TORCH_CHECK(!(upd && idx.has_value()), "rows can be picked without an update only");
+  TORCH_CHECK(!upd || (mix.has_value() && wout.has_value()), "an update needs mix and w_out");
+  at::Tensor xn = upd && x.dim() == 2 ? at::empty({T, S, (long)W}, x.options()) : x;
+  long rows = T;
+  if (idx) {
+    CHECK_CUDA(*idx);
+    TORCH_CHECK(idx->scalar_type() == at::kLong && idx->is_contiguous(), "idx must be int64");
+    rows = idx->numel();
+  }
+  c10::optional<at::Tensor> out;
+  if (w) out = at::empty({rows, (long)W}, x.options().dtype(out_dtype));
+  CHECK_RC(lk_stream_hyper_norm(x.data_ptr<float>(), x.stride(0), x.dim() == 3 ? W : 0, upd ? xn.data_ptr<float>() : nullptr, (int)S, ap, as, bp_, bs,
+                                yp, ys, ywp, top, upd ? fpo(mix, S * S, "mix") : nullptr, upd ? fpo(wout, S, "w_out") : nullptr, fpo(win, S, "w_in"),
+                                fpo(w, W, "norm weight"), (float)eps, (float)oscale, idx ? idx->data_ptr<int64_t>() : nullptr,
+                                out ? out->data_ptr() : nullptr, W, rows, W, esz, cur_stream()),
+           "stream_hyper_norm");
+  return {c10::optional<at::Tensor>(xn), out};
+}
+
+void relu_sq_(at::Tensor& x) {
+  CHECK_CUDA(x); CHECK_LASTDIM(x);
+  TORCH_CHECK(x.dim() == 2, "x must be 2-d");
+  CHECK_RC(lk_relu_sq_(x.data_ptr(), x.stride(0), x.size(0), (int)x.size(1), esz_of(x, "x"), cur_stream()), "relu_sq_");
+}
+
+at::Tensor gate_proj(const at::Tensor& h, const at::Tensor& w, const at::Tensor& bias, int64_t heads, double cap) {
+  CHECK_CUDA(h); CHECK_LASTDIM(h); CHECK_CUDA(w); CHECK_CONTIG(w);
+  same_type(w, h, "w");
+  TORCH_CHECK(h.dim() == 2 && w.dim() == 2 && w.size(1) == h.size(1) && w.size(0) == 2 * heads, "h [T, W], w [2 heads, W]");
+  at::Tensor out = at::empty({h.size(0), 2 * heads}, h.options().dtype(at::kFloat));
+  CHECK_RC(lk_gate_proj(h.data_ptr(), h.stride(0), w.data_ptr(), fp(bias, 2 * heads, "bias"), (int)(2 * heads), (int)h.size(1), h.size(0), (float)cap,
+                        out.data_ptr<float>(), esz_of(h, "h"), cur_stream()), "gate_proj");
+  return out;
+}
+
+std::vector<at::Tensor> router_choice(const at::Tensor& h, const at::Tensor& w, int64_t top, int64_t groups, int64_t keep, double scale, int64_t score,
+                                      const c10::optional<at::Tensor>& corr, int64_t gscore) {
+  CHECK_CUDA(h); CHECK_LASTDIM(h); CHECK_CUDA(w); CHECK_CONTIG(w);
+  same_type(w, h, "router");
+  TORCH_CHECK(h.dim() == 2 && w.dim() == 2 && w.size(1) == h.size(1), "h [T, W], router [E, W]");
+  const long T = h.size(0);
+  at::Tensor experts = at::empty({T, top}, h.options().dtype(at::kInt));
+  at::Tensor weights = at::empty({T, top}, h.options().dtype(at::kFloat));
+  CHECK_RC(lk_router_choice(h.data_ptr(), h.stride(0), w.data_ptr(), (int)w.size(0), (int)w.size(1), T, (int)top, (int)groups, (int)keep, (float)scale,
+                            (int)score, fpo(corr, w.size(0), "correction"), (int)gscore, experts.data_ptr<int>(), weights.data_ptr<float>(),
+                            esz_of(h, "h"), cur_stream()), "router_choice");
+  return {experts, weights};
+}
+
+at::Tensor mlstm_scan(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, const at::Tensor& gates, at::Tensor& S, at::Tensor& nm,
+                      const at::Tensor& cu, const at::Tensor& slots, const at::Tensor& positions, int64_t H, int64_t dk, int64_t dv, double q_scale,
+                      int64_t max_len) {
+  const long T = q.size(0);
+  TORCH_CHECK(H >= 1 && dk >= 1 && dk <= 256 && dv >= 1, "mlstm_scan sizes");
+  check_rows(q, T, H * dk, "q"); check_rows(k, T, H * dk, "k"); check_rows(v, T, H * dv, "v");
+  const int esz = esz_of(q, "q");
+  same_type(k, q, "k"); same_type(v, q, "v");
+  check_rows(gates, T, 2 * H, "gates");
+  CHECK_F32(gates);
+  check_seqs(cu, slots, positions, T);
+  CHECK_CUDA(S); CHECK_F32(S); CHECK_CONTIG(S); CHECK_CUDA(nm); CHECK_F32(nm); CHECK_CONTIG(nm);
+  TORCH_CHECK(S.dim() == 4 && S.size(1) == H && S.size(2) == dk && S.size(3) == dv, "state must be f32 [slots, H, dk, dv]");
+  TORCH_CHECK(nm.dim() == 4 && nm.size(0) == S.size(0) && nm.size(1) == H && nm.size(2) == (dv + 63) / 64 && nm.size(3) == dk + 4,
+              "normaliser must be f32 [slots, H, ceil(dv / 64), dk + 4]");
+  at::Tensor o = at::empty({T, H * dv}, q.options().dtype(at::kFloat));
+  CHECK_RC(lk_mlstm_scan(q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), esz, gates.data_ptr<float>(),
+                         gates.stride(0), (float)q_scale, S.data_ptr<float>(), nm.data_ptr<float>(), ip(cu), ip(slots), ip(positions),
+                         (int)(cu.numel() - 1), (int)H, (int)dk, (int)dv, o.data_ptr<float>(), o.stride(0), (int)max_len, cur_stream()),
+           "mlstm_scan");
+  return o;
+}
+
+void head_linear(const at::Tensor& x, const at::Tensor& w, int64_t x_head, at::Tensor& out) {
+  CHECK_CUDA(x); CHECK_LASTDIM(x); CHECK_CUDA(w); CHECK_CONTIG(w); CHECK_CUDA(out); CHECK_LASTDIM(out);
+  same_type(w, x, "w"); same_type(out, x, "out");
+  TORCH_CHECK(w.dim() == 3 && x.dim() == 2 && out.dim() == 3, "x [T, *], w [H, N, K], out [T, H, >= N]");
+  const long H = w.size(0), N = w.size(1), K = w.size(2);
+  TORCH_CHECK(x_head >= 0 && x.size(1) >= (H - 1) * x_head + K, "x has too few columns");
+  TORCH_CHECK(out.size(0) == x.size(0) && out.size(1) == H && out.size(2) >= N, "out must be [T, H, >= N]");
+  CHECK_RC(lk_head_linear(x.data_ptr(), x.stride(0), x_head, w.data_ptr(), (int)H, (int)N, (int)K, x.size(0), out.data_ptr(), out.stride(0),
+                          out.stride(1), esz_of(x, "x"), cur_stream()), "head_linear");
+}
+
+struct LatShapes { int H, KD, RP, BS, esz; const float* sink; };
+LatShapes lat_check(const at::Tensor& qa, const at::Tensor& cache, const at::Tensor& bt, const at::Tensor& ctx, const c10::optional<at::Tensor>& sink,
+                    int64_t rp, const at::Tensor& out) {
+  CHECK_CUDA(qa); CHECK_CUDA(cache); CHECK_CONTIG(cache); CHECK_CUDA(out); CHECK_CUDA(bt); CHECK_I32(bt); CHECK_LASTDIM(bt);
+  CHECK_CUDA(ctx); CHECK_I32(ctx); CHECK_CONTIG(ctx);
+  same_type(cache, qa, "cache"); same_type(out, qa, "out");
+  TORCH_CHECK(qa.dim() == 3 && cache.dim() == 3 && out.dim() == 3 && cache.size(2) == qa.size(2), "qa [T, H, KD], cache [blocks, BS, KD]");
+  TORCH_CHECK(qa.stride(2) == 1 && qa.stride(1) == qa.size(2) && out.stride(2) == 1 && out.stride(1) == rp, "heads must be adjacent");
+  TORCH_CHECK(out.size(0) == qa.size(0) && out.size(1) == qa.size(1) && out.size(2) == rp && rp < qa.size(2), "out must be [T, H, rp]");
+  TORCH_CHECK(bt.dim() == 2 && bt.size(0) == ctx.numel(), "block tables: one row per sequence");
+  return {(int)qa.size(1), (int)qa.size(2), (int)rp, (int)cache.size(1), esz_of(qa, "qa"), fpo(sink, qa.size(1), "sink")};
+}
+
+void latent_attn_prefill(const at::Tensor& qa, const at::Tensor& cache, const at::Tensor& bt, const at::Tensor& cu_q, const at::Tensor& ctx,
+                         int64_t window, double scale, const c10::optional<at::Tensor>& sink, int64_t rp, at::Tensor& out, int64_t max_len) {
+  const LatShapes s = lat_check(qa, cache, bt, ctx, sink, rp, out);
+  CHECK_CUDA(cu_q); CHECK_I32(cu_q); CHECK_CONTIG(cu_q);
+  TORCH_CHECK(cu_q.numel() == ctx.numel() + 1, "cu_q");
+  CHECK_RC(lk_latent_attn_prefill(qa.data_ptr(), qa.stride(0), cache.data_ptr(), ip(bt), (int)bt.stride(0), ip(cu_q), ip(ctx), (int)ctx.numel(),
+                                  qa.size(0), s.BS, s.H, s.KD, s.RP, (int)window, (float)scale, s.sink, out.data_ptr(), out.stride(0), s.esz,
+                                  cur_stream()), "latent_attn_prefill");
+}
+
+void latent_attn_decode(const at::Tensor& qa, const at::Tensor& cache, const at::Tensor& bt, const at::Tensor& ctx, int64_t window, double scale,
+                        const c10::optional<at::Tensor>& sink, int64_t rp, at::Tensor& out, int64_t splits) {
+  const LatShapes s = lat_check(qa, cache, bt, ctx, sink, rp, out);
+  TORCH_CHECK(ctx.numel() == qa.size(0) && splits >= 1, "one row per sequence");
+  at::Tensor part;
+  if (splits > 1) part = at::empty({qa.size(0) * s.H * splits * (rp + 2)}, qa.options().dtype(at::kFloat));
+  CHECK_RC(lk_latent_attn_decode(qa.data_ptr(), qa.stride(0), cache.data_ptr(), ip(bt), (int)bt.stride(0), ip(ctx), (int)qa.size(0), (int)splits, s.BS,
+                                 s.H, s.KD, s.RP, (int)window, (float)scale, s.sink, out.data_ptr(), out.stride(0),
+                                 splits > 1 ? part.data_ptr<float>() : nullptr, s.esz, cur_stream()), "latent_attn_decode");
+}
+
+at::Tensor latent_prep(const at::Tensor& u, int64_t dq, int64_t qr, const at::Tensor& wq, int64_t dkv, int64_t R, const c10::optional<at::Tensor>& wkv,
+                       int64_t rd, const at::Tensor& freq, const at::Tensor& positions, double eps, at::Tensor& cache, const at::Tensor& slots,
+                       int64_t rp) {
+  CHECK_CUDA(u); CHECK_LASTDIM(u); CHECK_CUDA(positions); CHECK_I32(positions); CHECK_CUDA(slots); CHECK_I32(slots);
+  CHECK_CUDA(cache); CHECK_CONTIG(cache); same_type(cache, u, "cache");
+  const long T = u.size(0);
+  TORCH_CHECK(u.dim() == 2 && dq >= 0 && u.size(1) >= dq + qr && (!wkv || (dkv >= 0 && u.size(1) >= dkv + R + rd)), "columns of u");
+  TORCH_CHECK(positions.numel() >= T && slots.numel() >= T && positions.is_contiguous() && slots.is_contiguous(), "positions / slots");
+  TORCH_CHECK(cache.dim() == 3, "cache [blocks, BS, KD]");
+  at::Tensor cq = at::empty({T, qr}, u.options());
+  CHECK_RC(lk_latent_prep(u.data_ptr(), u.stride(0), (int)dq, (int)qr, fp(wq, qr, "dq norm"), (int)dkv, (int)R, fpo(wkv, R, "dkv norm"), (int)rd,
+                          fp(freq, std::max<int64_t>(rd / 2, 1), "freq"), ip(positions), (float)eps, cache.data_ptr(), ip(slots), (int)rp,
+                          (int)cache.size(2), cq.data_ptr(), cq.stride(0), T, esz_of(u, "u"), cur_stream()), "latent_prep");
+  return cq;
+}
+
+void latent_query_rot(const at::Tensor& q, at::Tensor& qa, int64_t H, int64_t qdim, int64_t dim, int64_t rd, const at::Tensor& freq,
+                      const at::Tensor& positions, int64_t rp) {
+  CHECK_CUDA(q); CHECK_LASTDIM(q); CHECK_CUDA(qa); CHECK_LASTDIM(qa); same_type(qa, q, "qa");
+  CHECK_CUDA(positions); CHECK_I32(positions);
+  TORCH_CHECK(q.dim() == 2 && qa.dim() == 3 && qa.size(0) == q.size(0) && qa.size(1) == H && qa.stride(1) == qa.size(2) && q.size(1) >= H * qdim &&
+                  positions.numel() >= q.size(0), "q [T, H qdim], qa [T, H, KD]");
+  CHECK_RC(lk_latent_query_rot(q.data_ptr(), q.stride(0), qa.data_ptr(), qa.stride(0), (int)H, (int)qdim, (int)dim, (int)rd,
+                               fp(freq, std::max<int64_t>(rd / 2, 1), "freq"), ip(positions), (int)rp, (int)qa.size(2), q.size(0), esz_of(q, "q"),
+                               cur_stream()), "latent_query_rot");
+}
+
 }  // namespace
 // build provenance: "LKSTAMP:<hash of sources + flags>", generated by csrc/build.py at link time
 extern "C" const char lk_source_stamp[];
@@ -1790,6 +1970,16 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gemm_grouped", &gemm_grouped);
   m.def("gemm_grouped_supported", [](int64_t N, int64_t K, bool swiglu) { return lk_gemm_grouped_supported((int)N, (int)K, swiglu ? 1 : 0) != 0; });
   m.def("moe_gemm", &moe_gemm);
+  m.def("stream_hyper_norm", &stream_hyper_norm);
+  m.def("relu_sq_", &relu_sq_);
+  m.def("gate_proj", &gate_proj);
+  m.def("router_choice", &router_choice);
+  m.def("mlstm_scan", &mlstm_scan);
+  m.def("head_linear", &head_linear);
+  m.def("latent_attn_prefill", &latent_attn_prefill);
+  m.def("latent_attn_decode", &latent_attn_decode);
+  m.def("latent_prep", &latent_prep);
+  m.def("latent_query_rot", &latent_query_rot);
   m.def("window_mark", [](int64_t id) { CHECK_RC(lk_window_mark((int)id, cur_stream()), "window_mark"); });
   m.def("debug_invalid_launch", []() { CHECK_RC(lk_debug_invalid_launch(cur_stream()), "debug_invalid_launch"); });
   // a HIP stream restricted to the CUs of a bit mask (32 CUs per word): two kernels that

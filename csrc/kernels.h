@@ -329,3 +329,38 @@ int lk_sigmoid_mul_(void* x, long xs, const void* g, long gs, long rows, int n, 
 int lk_moe_route(const int* ids, const int* table, int vocab, int top, int E, int T, int* seg, int* order, hipStream_t st);
 int lk_moe_gemm(const void* x, long xs, const int* order, const int* seg, int E, int top, long pairs, const void* w, int N, int K,
                 int act, void* out, long os, int esz, hipStream_t st);
+
+// csrc/hyper_stream.hip: a residual stream of S mixed copies: sublayer result in, next combination and its layer norm out; squared relu
+int lk_stream_hyper_norm(const float* xin, long xrow, long xstr, float* xout, int S, const void* a, long as, const void* b, long bs,
+                         const void* y, long ys, const float* yw, int top, const float* mix, const float* wout, const float* win,
+                         const float* w, float eps, float oscale, const long* idx, void* out, long os, long rows, int W, int esz,
+                         hipStream_t st);
+int lk_relu_sq_(void* x, long xs, long rows, int n, int esz, hipStream_t st);
+
+// csrc/row_proj.hip: skinny f32-result projections: gates of a gated recurrence, router choice with weights
+int lk_gate_proj(const void* h, long hs, const void* w, const float* bias, int N, int K, long rows, float cap, float* out, int esz,
+                 hipStream_t st);
+int lk_router_choice(const void* h, long hs, const void* w, int E, int K, long rows, int top, int groups, int keep, float scale, int score,
+                     const float* corr, int gscore, int* experts, float* weights, int esz, hipStream_t st);
+
+// csrc/mlstm.hip: matrix memory with exponential gates (S [slots, H, dk, dv], n | m [slots, H, ceil(dv / 64), dk + 4])
+int lk_mlstm_scan(const void* q, long qs, const void* k, long ks, const void* v, long vs, int esz, const float* gates, long gs, float q_scale,
+                  float* S, float* nm, const int* cu, const int* slots, const int* positions, int seqs, int H, int dk, int dv, float* o,
+                  long os, int max_len, hipStream_t st);
+
+// csrc/head_linear.hip: out[t, h, :N] = w[h] x[t, h xh : h xh + K]
+int lk_head_linear(const void* x, long xs, long xh, const void* w, int H, int N, int K, long rows, void* out, long os, long oh, int esz,
+                   hipStream_t st);
+
+// csrc/latent_attn.hip: attention over a cached latent shared by all heads (cache [blocks, BS, KD], row = latent | rotated part) and
+// the preparation of its operands
+int lk_latent_attn_prefill(const void* q, long qs, const void* cache, const int* bt, int bt_stride, const int* cu_q, const int* ctx_lens, int nseq,
+                           long rows, int BS, int H, int KD, int RP, int window, float scale, const float* sink, void* out, long os, int esz,
+                           hipStream_t st);
+int lk_latent_attn_decode(const void* q, long qs, const void* cache, const int* bt, int bt_stride, const int* ctx_lens, int B, int Z, int BS, int H,
+                          int KD, int RP, int window, float scale, const float* sink, void* out, long os, float* part, int esz, hipStream_t st);
+int lk_latent_prep(const void* u, long us, int dq, int qr, const float* wq, int dkv, int R, const float* wkv, int rd, const float* freq,
+                   const int* positions, float eps, void* cache, const int* slots, int RP, int KD, void* cq, long cqs, long rows, int esz,
+                   hipStream_t st);
+int lk_latent_query_rot(const void* q, long qs, void* qa, long as, int H, int qdim, int dim, int rd, const float* freq, const int* positions, int RP,
+                        int KD, long rows, int esz, hipStream_t st);

@@ -1,0 +1,426 @@
+// Matrix memory with exponential gates: per head and sequence, from log input gates i_t and log forget gates f_t,
+//
+//   m_t = max(f_t + m_(t-1), i_t)                                   m_0 = 0
+//   S_t = exp(f_t + m_(t-1) - m_t) S_(t-1) + exp(i_t - m_t) k_t v_t^T          n_t likewise with k_t alone
+//   o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6)
+//
+// q, k, v rows in bf16 or f32; gates, state and everything in between f32.  S [slots, H, dk, dv]; beside it n and m, one copy per
+// block of 64 state columns ([slots, H, Z, dk + 4], m behind n), since the workgroups of a head run independently.
+//
+// A batch is a list of sequences (prompt portions of any length, decode rows of length 1): rows [cu[s], cu[s+1]) belong to
+// sequence s, whose state lives in slot slots[s] (< 0: a padding row, its output rows are zeroed) and starts from zero when its
+// first row sits at position 0.
+#include "common.h"
+#include "kernels.h"
+
+namespace {
+
+template <typename T>
+LK_DEVICE float ldf(const T* p);
+template <>
+LK_DEVICE float ldf<bf16_t>(const bf16_t* p) { return bf2f(*p); }
+template <>
+LK_DEVICE float ldf<float>(const float* p) { return *p; }
+
+constexpr int kColBlock = 64;    // state columns of a workgroup
+constexpr int kChunkMin = 8;     // from this many rows of some sequence on: the chunked form
+constexpr float kDenEps = 1e-6f;
+
+struct MlstmParams {
+  const void* q;
+  const void* k;
+  const void* v;
+  long qs, ks, vs;
+  const float* gates;  // rows of 2 H: log input gates, log forget gates
+  long gs;
+  float q_scale;
+  float* S;
+  float* nm;
+  const int* cu;
+  const int* slots;
+  const int* positions;
+  float* o;
+  long os;
+  int H, dk, dv, Z;
+};
+
+LK_DEVICE void zero_rows(const MlstmParams& a, int row0, int len, int h, int j0, int nthreads) {
+  for (int i = threadIdx.x; i < len * kColBlock; i += nthreads) {
+    const int c = j0 + i % kColBlock;
+    if (c < a.dv) a.o[(long)(row0 + i / kColBlock) * a.os + (long)h * a.dv + c] = 0.f;
+  }
+}
+
+// ---- token by token (decode rows, very short portions): the state streams through registers once per step.
+// grid (sequence, head, column block).  256 threads = 16 groups of 4 adjacent columns x 16 row slices; a thread holds the rows
+// rs, rs + 16, ... of its 4 columns (16-byte accesses, VEC).
+template <typename T, int NR, bool VEC>
+__global__ __launch_bounds__(256) void mlstm_step_kernel(MlstmParams a) {
+  __shared__ float sq[NR * 16], sk[NR * 16], red[4][16][5];
+  const int s = blockIdx.x, h = blockIdx.y, z = blockIdx.z, j0 = z * kColBlock, tid = threadIdx.x;
+  const int row0 = a.cu[s], len = a.cu[s + 1] - row0, slot = a.slots[s];
+  if (len <= 0) return;
+  if (slot < 0) {
+    zero_rows(a, row0, len, h, j0, 256);
+    return;
+  }
+  const int cg = tid & 15, rs = tid >> 4, wv = tid >> 6, lane = tid & 63, c0 = j0 + 4 * cg;
+  const bool fresh = a.positions[row0] == 0;
+  float* Sg = a.S + ((long)slot * a.H + h) * a.dk * a.dv + c0;
+  float* nmg = a.nm + (((long)slot * a.H + h) * a.Z + z) * (a.dk + 4);
+  floatx4 S[NR];
+  float n[NR];
+#pragma unroll
+  for (int ii = 0; ii < NR; ++ii) {
+    const int i = rs + 16 * ii;
+    S[ii] = floatx4{0.f, 0.f, 0.f, 0.f};
+    n[ii] = 0.f;
+    if (!fresh && i < a.dk) {
+      n[ii] = nmg[i];
+      if constexpr (VEC) {
+        if (c0 < a.dv) S[ii] = *reinterpret_cast<const floatx4*>(Sg + (long)i * a.dv);
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (c0 + e < a.dv) S[ii][e] = Sg[(long)i * a.dv + e];
+      }
+    }
+  }
+  float m = fresh ? 0.f : nmg[a.dk];
+  const T* qg = reinterpret_cast<const T*>(a.q) + (long)h * a.dk;
+  const T* kg = reinterpret_cast<const T*>(a.k) + (long)h * a.dk;
+  const T* vg = reinterpret_cast<const T*>(a.v) + (long)h * a.dv;
+  for (int t = 0; t < len; ++t) {
+    const long row = row0 + t;
+    __syncthreads();   // the previous token's operands and sums have been read
+    for (int i = tid; i < NR * 16; i += 256) {
+      sq[i] = i < a.dk ? ldf<T>(qg + row * a.qs + i) * a.q_scale : 0.f;
+      sk[i] = i < a.dk ? ldf<T>(kg + row * a.ks + i) : 0.f;
+    }
+    float v[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = c0 + e < a.dv ? ldf<T>(vg + row * a.vs + c0 + e) : 0.f;
+    const float ig = a.gates[row * a.gs + h], fg = a.gates[row * a.gs + a.H + h];
+    const float mn = fmaxf(fg + m, ig), fa = expf(fg + m - mn), ia = expf(ig - mn);
+    m = mn;
+    __syncthreads();
+    float acc[5] = {0.f, 0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ii = 0; ii < NR; ++ii) {
+      const int i = rs + 16 * ii;
+      const float kk = ia * sk[i], qq = sq[i];
+      n[ii] = fa * n[ii] + kk;
+      acc[4] += n[ii] * qq;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        S[ii][e] = fa * S[ii][e] + kk * v[e];
+        acc[e] += S[ii][e] * qq;
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < 5; ++e) {
+      acc[e] += __shfl_xor(acc[e], 16, 64);
+      acc[e] += __shfl_xor(acc[e], 32, 64);
+    }
+    if (lane < 16) {
+#pragma unroll
+      for (int e = 0; e < 5; ++e) red[wv][lane][e] = acc[e];
+    }
+    __syncthreads();
+    if (tid < 64) {   // thread = (column group, column in it)
+      const int g4 = tid >> 2, e = tid & 3;
+      const float num = (red[0][g4][e] + red[1][g4][e]) + (red[2][g4][e] + red[3][g4][e]);
+      const float nq = (red[0][g4][4] + red[1][g4][4]) + (red[2][g4][4] + red[3][g4][4]);
+      const int c = j0 + tid;
+      if (c < a.dv) a.o[row * a.os + (long)h * a.dv + c] = num / (fmaxf(fabsf(nq), expf(-m)) + kDenEps);
+    }
+  }
+#pragma unroll
+  for (int ii = 0; ii < NR; ++ii) {
+    const int i = rs + 16 * ii;
+    if (i < a.dk) {
+      if constexpr (VEC) {
+        if (c0 < a.dv) *reinterpret_cast<floatx4*>(Sg + (long)i * a.dv) = S[ii];
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (c0 + e < a.dv) Sg[(long)i * a.dv + e] = S[ii][e];
+      }
+      if (cg == 0) nmg[i] = n[ii];
+    }
+  }
+  if (tid == 0) nmg[a.dk] = m;
+}
+
+// ---- chunked matrix form (prompt portions): the recurrence unrolled over chunks of 16 tokens, products on true-f32 MFMAs
+// (bf16 rows: the q.k products on bf16 MFMAs, exact products either way), the state in the accumulators' layout from
+// chunk to chunk.  With F_t = f_1 + .. + f_t inside the chunk, S, n, m the state before it, a_s = i_s - F_s:
+//   m_t = F_t + max(m, max_{s<=t} a_s)
+//   D_ts = exp(F_t + a_s - m_t)  (s <= t),     e_t = exp(F_t + m - m_t)
+//   num_t = e_t S^T q_t + sum_s D_ts (q_t.k_s) v_s,      nq_t = e_t n.q_t + sum_s D_ts (q_t.k_s)
+//   S' = e_L S + sum_s D_Ls k_s v_s^T,   n' = e_L n + sum_s D_Ls k_s,   m' = m_L
+// Tokens past the end of the last chunk get f = 0, i = -1e30: they neither decay nor feed the state.
+// grid (sequence, head, column block): wave w owns the 16 state columns j0 + 16 w .. + 15 (all dk rows: NR accumulator tiles).
+template <typename T, int NR>
+__global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a) {
+  constexpr int NP = NR * 16, LD = NP + 4, L = 16, EV = 16 / sizeof(T), LH = NP + 8;
+  constexpr bool BF = sizeof(T) == 2 && NP % 32 == 0;
+  __shared__ __attribute__((aligned(16))) float sk[L][LD];
+  __shared__ __attribute__((aligned(16))) float sq[L][LD];
+  __shared__ __attribute__((aligned(16))) bf16_t hk[BF ? L : 1][BF ? LH : 8];   // the raw bf16 rows (q.k products)
+  __shared__ __attribute__((aligned(16))) bf16_t hq[BF ? L : 1][BF ? LH : 8];
+  __shared__ float sv[L][kColBlock], sn[2][NP], si[L], sf[L];
+  const int s = blockIdx.x, h = blockIdx.y, z = blockIdx.z, tid = threadIdx.x, j0 = z * kColBlock;
+  const int lane = tid & 63, w = tid >> 6, n16 = lane & 15, g = lane >> 4;
+  const int col = j0 + 16 * w + n16;
+  const bool cv = col < a.dv;
+  const int row0 = a.cu[s], len = a.cu[s + 1] - row0, slot = a.slots[s];
+  if (len <= 0) return;
+  if (slot < 0) {
+    zero_rows(a, row0, len, h, j0, 256);
+    return;
+  }
+  const bool fresh = a.positions[row0] == 0;
+  float* Sg = a.S + ((long)slot * a.H + h) * a.dk * a.dv + (cv ? col : 0);
+  float* nmg = a.nm + (((long)slot * a.H + h) * a.Z + z) * (a.dk + 4);
+  floatx4 S[NR];
+#pragma unroll
+  for (int nt = 0; nt < NR; ++nt)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int i = nt * 16 + 4 * g + j;
+      S[nt][j] = (!fresh && cv && i < a.dk) ? Sg[(long)i * a.dv] : 0.f;
+    }
+  float m = fresh ? 0.f : nmg[a.dk];
+  for (int i = tid; i < NP; i += 256) sn[0][i] = (!fresh && i < a.dk) ? nmg[i] : 0.f;
+  const T* qg = reinterpret_cast<const T*>(a.q) + (long)h * a.dk;
+  const T* kg = reinterpret_cast<const T*>(a.k) + (long)h * a.dk;
+  const T* vg = reinterpret_cast<const T*>(a.v) + (long)h * a.dv;
+  const bool vec = a.dk % EV == 0 && a.qs % EV == 0 && a.ks % EV == 0 && (reinterpret_cast<uintptr_t>(qg) & 15) == 0 &&
+                   (reinterpret_cast<uintptr_t>(kg) & 15) == 0;
+  // the next chunk's operands are requested before this chunk's products are issued
+  constexpr int CPR = NP / EV, NPF = (2 * L * CPR + 255) / 256;
+  uint4_t pre[NPF];
+  float prev_[4], prei = 0.f, pref = 0.f;
+  auto fetch = [&](int t0) {
+    const int tl = min(L, len - t0), ncpr = a.dk / EV;
+#pragma unroll
+    for (int x = 0; x < NPF; ++x) {
+      const int i = tid + 256 * x;
+      pre[x] = uint4_t{0u, 0u, 0u, 0u};
+      if (i < 2 * L * CPR) {
+        const int which = i / (L * CPR), r = i % (L * CPR), t = r / CPR, c = r % CPR;
+        if (t < tl && c < ncpr)
+          pre[x] = *reinterpret_cast<const uint4_t*>((which ? qg + (long)(row0 + t0 + t) * a.qs : kg + (long)(row0 + t0 + t) * a.ks) + c * EV);
+      }
+    }
+#pragma unroll
+    for (int x = 0; x < 4; ++x) {
+      const int i = tid + 256 * x, t = i >> 6, c = i & 63;
+      prev_[x] = (t < tl && j0 + c < a.dv) ? ldf<T>(vg + (long)(row0 + t0 + t) * a.vs + j0 + c) : 0.f;
+    }
+    if (tid < L) {
+      prei = tid < tl ? a.gates[(long)(row0 + t0 + tid) * a.gs + h] : -1e30f;
+      pref = tid < tl ? a.gates[(long)(row0 + t0 + tid) * a.gs + a.H + h] : 0.f;
+    }
+  };
+  fetch(0);
+  int cur = 0;
+  for (int t0 = 0; t0 < len; t0 += L) {
+    const int tl = min(L, len - t0);
+    __syncthreads();   // the previous chunk has been consumed
+    if (vec) {
+#pragma unroll
+      for (int x = 0; x < NPF; ++x) {
+        const int i = tid + 256 * x;
+        if (i < 2 * L * CPR) {
+          const int which = i / (L * CPR), r = i % (L * CPR), t = r / CPR, c = r % CPR;
+          float* dst = (which ? sq[t] : sk[t]) + c * EV;
+          if constexpr (sizeof(T) == 2) {
+            const short8 v = __builtin_bit_cast(short8, pre[x]);
+            const float f = which ? a.q_scale : 1.f;
+            *reinterpret_cast<floatx4*>(dst) = floatx4{bf2f((bf16_t)v[0]) * f, bf2f((bf16_t)v[1]) * f, bf2f((bf16_t)v[2]) * f, bf2f((bf16_t)v[3]) * f};
+            *reinterpret_cast<floatx4*>(dst + 4) = floatx4{bf2f((bf16_t)v[4]) * f, bf2f((bf16_t)v[5]) * f, bf2f((bf16_t)v[6]) * f, bf2f((bf16_t)v[7]) * f};
+            if constexpr (BF) *reinterpret_cast<uint4_t*>((which ? hq[t] : hk[t]) + c * EV) = pre[x];
+          } else {
+            const floatx4 v = __builtin_bit_cast(floatx4, pre[x]);
+            const float f = which ? a.q_scale : 1.f;
+            *reinterpret_cast<floatx4*>(dst) = floatx4{v[0] * f, v[1] * f, v[2] * f, v[3] * f};
+          }
+        }
+      }
+    } else {
+      for (int i = tid; i < 2 * L * NP; i += 256) {
+        const int which = i / (L * NP), r = i % (L * NP), t = r / NP, c = r % NP;
+        const bool in = t < tl && c < a.dk;
+        const long row = row0 + t0 + t;
+        T raw = T(0);
+        if (in) raw = which ? qg[row * a.qs + c] : kg[row * a.ks + c];
+        (which ? sq[t] : sk[t])[c] = ldf<T>(&raw) * (which ? a.q_scale : 1.f);
+        if constexpr (BF) (which ? hq[t] : hk[t])[c] = raw;
+      }
+    }
+#pragma unroll
+    for (int x = 0; x < 4; ++x) {
+      const int i = tid + 256 * x;
+      sv[i >> 6][i & 63] = prev_[x];
+    }
+    if (tid < L) {
+      si[tid] = prei;
+      sf[tid] = pref;
+    }
+    __syncthreads();
+    if (t0 + L < len) fetch(t0 + L);
+    // inside every 16-lane group: lane t ends up with F_t and max_{s<=t} a_s
+    float F = sf[n16];
+#pragma unroll
+    for (int o = 1; o < 16; o <<= 1) {
+      const float v = __shfl_up(F, o, 16);
+      if (n16 >= o) F += v;
+    }
+    const float as = si[n16] - F;
+    float am = as;
+#pragma unroll
+    for (int o = 1; o < 16; o <<= 1) {
+      const float v = __shfl_up(am, o, 16);
+      if (n16 >= o) am = fmaxf(am, v);
+    }
+    const float mt = F + fmaxf(m, am);          // m_t of t = n16
+    const float et = expf(F + m - mt);
+    const float Fl = __shfl(F, 15, 16), ml = __shfl(mt, 15, 16);
+    // G^T: lane (t = n16, g) gets G[t][s = 4g + j] = q_t . k_s
+    floatx4 gt = {0.f, 0.f, 0.f, 0.f};
+    if constexpr (BF) {
+#pragma unroll
+      for (int nb = 0; nb < NP / 32; ++nb) {
+        const short8 ka = *reinterpret_cast<const short8*>(&hk[n16][nb * 32 + 8 * g]);
+        const short8 qb = *reinterpret_cast<const short8*>(&hq[n16][nb * 32 + 8 * g]);
+        gt = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ka, qb, gt, 0, 0, 0);
+      }
+#pragma unroll
+      for (int j = 0; j < 4; ++j) gt[j] *= a.q_scale;
+    } else {
+#pragma unroll
+      for (int nb = 0; nb < NR; ++nb) {
+        const floatx4 a4 = *reinterpret_cast<const floatx4*>(&sk[n16][nb * 16 + 4 * g]);
+        const floatx4 b4 = *reinterpret_cast<const floatx4*>(&sq[n16][nb * 16 + 4 * g]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) gt = __builtin_amdgcn_mfma_f32_16x16x4f32(a4[j], b4[j], gt, 0, 0, 0);
+      }
+    }
+    float M[4], xv[4], wl[4], ms = 0.f;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int sj = 4 * g + j;
+      const float a_s = __shfl(as, sj, 16);
+      M[j] = sj <= n16 ? gt[j] * expf(F + a_s - mt) : 0.f;
+      ms += M[j];
+      xv[j] = sv[sj][16 * w + n16];
+      wl[j] = expf(Fl + a_s - ml);
+    }
+    // num: rows t = 4g + j, column n16 of this wave's tile; n . q of t = n16 beside it
+    floatx4 ya = {0.f, 0.f, 0.f, 0.f};
+    float nq = 0.f;
+#pragma unroll
+    for (int nt = 0; nt < NR; ++nt) {
+      const floatx4 q4 = *reinterpret_cast<const floatx4*>(&sq[n16][nt * 16 + 4 * g]);
+      const floatx4 n4 = *reinterpret_cast<const floatx4*>(&sn[cur][nt * 16 + 4 * g]);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        ya = __builtin_amdgcn_mfma_f32_16x16x4f32(q4[j], S[nt][j], ya, 0, 0, 0);
+        nq += q4[j] * n4[j];
+      }
+    }
+    nq = et * nq + ms;   // e_t is the same in the four lane groups of t
+    // (each group holds its quarter of both sums: e_t distributes over them)
+    nq += __shfl_xor(nq, 16, 64);
+    nq += __shfl_xor(nq, 32, 64);
+    const float rden = 1.f / (fmaxf(fabsf(nq), expf(-mt)) + kDenEps);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) ya[j] *= __shfl(et, 4 * g + j, 16);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) ya = __builtin_amdgcn_mfma_f32_16x16x4f32(M[j], xv[j], ya, 0, 0, 0);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int t = 4 * g + j;
+      const float rd = __shfl(rden, t, 16);
+      if (cv && t < tl) a.o[(long)(row0 + t0 + t) * a.os + (long)h * a.dv + col] = ya[j] * rd;
+    }
+    // state: rows i = 16 nt + 4g + j, column n16
+    const float dec = expf(Fl + m - ml);
+#pragma unroll
+    for (int nt = 0; nt < NR; ++nt) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) S[nt][j] *= dec;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        S[nt] = __builtin_amdgcn_mfma_f32_16x16x4f32(sk[4 * g + j][nt * 16 + n16] * wl[j], xv[j], S[nt], 0, 0, 0);
+    }
+    float ws[L];         // D_Ls of every s, uniform
+#pragma unroll
+    for (int x = 0; x < L; ++x) ws[x] = __shfl(wl[x & 3], 16 * (x >> 2), 64);
+    for (int i = tid; i < NP; i += 256) {
+      float v = dec * sn[cur][i];
+#pragma unroll
+      for (int x = 0; x < L; ++x) v += ws[x] * sk[x][i];
+      sn[cur ^ 1][i] = v;
+    }
+    cur ^= 1;
+    m = ml;
+  }
+  __syncthreads();
+  if (cv) {
+#pragma unroll
+    for (int nt = 0; nt < NR; ++nt)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int i = nt * 16 + 4 * g + j;
+        if (i < a.dk) Sg[(long)i * a.dv] = S[nt][j];
+      }
+  }
+  for (int i = tid; i < a.dk; i += 256) nmg[i] = sn[cur][i];
+  if (tid == 0) nmg[a.dk] = m;
+}
+
+template <typename T>
+int scan_t(const MlstmParams& a, int S, int max_len, hipStream_t st) {
+  const dim3 grid((unsigned)S, (unsigned)a.H, (unsigned)a.Z);
+  if (max_len >= kChunkMin) {
+#define LK_CHUNK(NR) mlstm_chunk_kernel<T, NR><<<grid, 256, 0, st>>>(a)
+    if (a.dk <= 16) LK_CHUNK(1);
+    else if (a.dk <= 32) LK_CHUNK(2);
+    else if (a.dk <= 64) LK_CHUNK(4);
+    else if (a.dk <= 128) LK_CHUNK(8);
+    else if (a.dk <= 256) LK_CHUNK(16);
+    else return -1;
+#undef LK_CHUNK
+  } else {
+    const bool vec = a.dv % 4 == 0 && reinterpret_cast<uintptr_t>(a.S) % 16 == 0;
+#define LK_STEP(NR)                                               \
+  if (vec) mlstm_step_kernel<T, NR, true><<<grid, 256, 0, st>>>(a); \
+  else mlstm_step_kernel<T, NR, false><<<grid, 256, 0, st>>>(a)
+    if (a.dk <= 16) { LK_STEP(1); }
+    else if (a.dk <= 32) { LK_STEP(2); }
+    else if (a.dk <= 64) { LK_STEP(4); }
+    else if (a.dk <= 128) { LK_STEP(8); }
+    else if (a.dk <= 256) { LK_STEP(16); }
+    else return -1;
+#undef LK_STEP
+  }
+  LK_CHECK_LAUNCH();
+  return 0;
+}
+
+}  // namespace
+
+int lk_mlstm_scan(const void* q, long qs, const void* k, long ks, const void* v, long vs, int esz, const float* gates, long gs, float q_scale,
+                  float* S, float* nm, const int* cu, const int* slots, const int* positions, int seqs, int H, int dk, int dv, float* o,
+                  long os, int max_len, hipStream_t st) {
+  if (seqs <= 0) return 0;
+  if (H < 1 || H > 65535 || dk < 1 || dk > 256 || dv < 1 || (dv + kColBlock - 1) / kColBlock > 65535) return -1;
+  MlstmParams a;
+  a.q = q; a.k = k; a.v = v; a.qs = qs; a.ks = ks; a.vs = vs; a.gates = gates; a.gs = gs; a.q_scale = q_scale; a.S = S; a.nm = nm;
+  a.cu = cu; a.slots = slots; a.positions = positions; a.o = o; a.os = os; a.H = H; a.dk = dk; a.dv = dv;
+  a.Z = (dv + kColBlock - 1) / kColBlock;
+  return esz == 2 ? scan_t<bf16_t>(a, seqs, max_len, st) : scan_t<float>(a, seqs, max_len, st);
+}

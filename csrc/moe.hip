@@ -53,17 +53,6 @@ __global__ __launch_bounds__(kRouteThreads) void moe_route_kernel(const int* __r
   for (int p = threadIdx.x; p < n; p += kRouteThreads) order[atomicAdd(&nxt[expert_of(p)], 1)] = p;
 }
 
-// 16 bytes of row `r` at element k (EV elements; zeros past K): one vector load when the row allows it
-template <typename T>
-LK_DEVICE uint4_t frag(const T* r, int k, int K, bool vec) {
-  constexpr int EV = El<T>::V;
-  if (vec && k + EV <= K) return ld16(r + k);
-  alignas(16) T tmp[EV];
-#pragma unroll
-  for (int e = 0; e < EV; ++e) tmp[e] = k + e < K ? r[k + e] : T(0);
-  return *reinterpret_cast<const uint4_t*>(tmp);
-}
-
 // grid (row tiles of 16 RT pairs: at most pairs / (16 RT) + E, column blocks): 4 waves side by side along the columns, each
 // RT row tiles x NB column tiles of 16 x 16 in registers, so a step of the contraction costs RT + NB fragment loads for
 // RT x NB MFMAs (RT = 1, NB = 2: decode-sized steps, where the experts' weights are read once and little else
