@@ -1846,10 +1846,12 @@ at::Tensor mlstm_scan(const at::Tensor& q, const at::Tensor& k, const at::Tensor
   TORCH_CHECK(S.dim() == 4 && S.size(1) == H && S.size(2) == dk && S.size(3) == dv, "state must be f32 [slots, H, dk, dv]");
   TORCH_CHECK(nm.dim() == 4 && nm.size(0) == S.size(0) && nm.size(1) == H && nm.size(2) == (dv + 63) / 64 && nm.size(3) == dk + 4,
               "normaliser must be f32 [slots, H, ceil(dv / 64), dk + 4]");
-  at::Tensor o = at::empty({T, H * dv}, q.options().dtype(at::kFloat));
+  at::Tensor o = at::empty({T, H * dv}, q.options().dtype(at::kFloat)), pre;
+  if (max_len >= lk_mlstm_chunk_min()) pre = at::empty({T, H, 4}, q.options().dtype(at::kFloat));
   CHECK_RC(lk_mlstm_scan(q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), esz, gates.data_ptr<float>(),
                          gates.stride(0), (float)q_scale, S.data_ptr<float>(), nm.data_ptr<float>(), ip(cu), ip(slots), ip(positions),
-                         (int)(cu.numel() - 1), (int)H, (int)dk, (int)dv, o.data_ptr<float>(), o.stride(0), (int)max_len, cur_stream()),
+                         (int)(cu.numel() - 1), (int)H, (int)dk, (int)dv, o.data_ptr<float>(), o.stride(0), (int)max_len,
+                         pre.defined() ? pre.data_ptr<float>() : nullptr, cur_stream()),
            "mlstm_scan");
   return o;
 }

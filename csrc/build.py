@@ -29,15 +29,9 @@ BUILD = ROOT / "build" / "csrc"
 PKG = ROOT / "llm_kubernetes_minikube_sharp4dev_amd"
 ARCH = os.environ.get("LK_OFFLOAD_ARCH", "gfx950")
 EXT_NAME = "_C"
-# Kernel files generated without packed-f32 instructions (v_pk_add / mul / fma_f32): plain f32 code
-# keeps its scalar VALU forms (the host pass warns that it does not know the feature).  The older
-# files keep the code generation their bit-exact fused-vs-unfused tests were written against (the
-# flag moves single roundings in the fused RoPE epilogue: tests/test_kernels_gpu.py
-# test_ws_linear_rope_kv_matches_unfused).
+# Every kernel file is generated without packed-f32 instructions (v_pk_add / mul / fma_f32): f32 code keeps its scalar VALU
+# forms (the host pass warns that it does not know the feature).
 NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
-NO_PACKED_FILES = ("attn_sigmoid.hip", "ssm.hip", "stream_f32.hip", "stream_ln.hip", "delta_scan.hip", "attn_sink.hip",
-                   "window_ops.hip", "moe.hip", "parallel_ops.hip", "hyper_stream.hip", "row_proj.hip", "mlstm.hip",
-                   "head_linear.hip", "latent_attn.hip")
 
 
 def _torch_paths():
@@ -71,8 +65,7 @@ def _codegen_flags(debug: bool = False) -> tuple[list[str], list[str]]:
     common = ["-O3", "-fPIC", "-std=c++17"]
     if debug:
         common += ["-DLK_DEBUG", "-g"]
-    kern = common + [f"--offload-arch={ARCH}", "-munsafe-fp-atomics", "-ffp-contract=fast", "|", *NO_PACKED_FILES,
-                     *NO_PACKED_FP32]
+    kern = common + [f"--offload-arch={ARCH}", "-munsafe-fp-atomics", "-ffp-contract=fast", *NO_PACKED_FP32]
     bind = common + [f"--offload-arch={ARCH}", "-DTORCH_API_INCLUDE_EXTENSION_H", f"-DTORCH_EXTENSION_NAME={EXT_NAME}",
                      "-DUSE_ROCM=1", "-D__HIP_PLATFORM_AMD__=1"]
     return kern, bind
@@ -112,7 +105,7 @@ def build(clean: bool = False, jobs: int | None = None, verbose: bool = False, d
     common = ["-O3", "-fPIC", "-std=c++17", f"-D_GLIBCXX_USE_CXX11_ABI={abi}", f"-I{CSRC}"]
     if debug:
         common += ["-DLK_DEBUG", "-g"]
-    kern_flags = common + [f"--offload-arch={ARCH}", "-munsafe-fp-atomics", "-ffp-contract=fast"]
+    kern_flags = common + [f"--offload-arch={ARCH}", "-munsafe-fp-atomics", "-ffp-contract=fast", *NO_PACKED_FP32]
     bind_flags = common + [
         f"--offload-arch={ARCH}",
         "-DTORCH_API_INCLUDE_EXTENSION_H",
@@ -127,8 +120,7 @@ def build(clean: bool = False, jobs: int | None = None, verbose: bool = False, d
     jobs_list = []
     for src in sorted(CSRC.glob("*.hip")):
         obj = BUILD / (src.stem + ".o")
-        extra = NO_PACKED_FP32 if src.name in NO_PACKED_FILES else []
-        jobs_list.append((src, obj, [hipcc, *kern_flags, *extra, "-c", str(src), "-o", str(obj)]))
+        jobs_list.append((src, obj, [hipcc, *kern_flags, "-c", str(src), "-o", str(obj)]))
     bsrc = CSRC / "bindings.cpp"
     bobj = BUILD / "bindings.o"
     jobs_list.append((bsrc, bobj, [hipcc, *bind_flags, "-x", "hip", "-c", str(bsrc), "-o", str(bobj)]))

@@ -2,22 +2,22 @@
 // projections between a head's own space and a latent that all heads share.
 //
 // Computed transposed (A = weight rows, B = token rows), so a lane ends up with 4 adjacent output columns of one token: one 8- or
-// 16-byte store.  grid (token tiles, column tiles, heads); 4 waves side by side along the tokens, each RT tiles of 16 tokens x 4
-// tiles of 16 columns; fragments straight from memory (the weights of a head and column tile are read by every wave: L1 / L2).
+// 16-byte store.  grid (token tiles, column tiles, heads); 4 waves as WT x (4 / WT) along tokens x columns, each RT tiles of 16
+// tokens x 4 tiles of 16 columns; fragments straight from memory (what the waves of a workgroup share is an L1 hit).
 #include "common.h"
 #include "kernels.h"
 #include "attn_frag.h"
 
 namespace {
 
-template <typename T, int RT>
+template <typename T, int RT, int WT>
 __global__ __launch_bounds__(256) void head_linear_kernel(const T* __restrict__ x, long xs, long xh, const T* __restrict__ w, int N, int K,
                                                           long rows, T* __restrict__ out, long os, long oh, int vec, int vst) {
-  constexpr int EV = El<T>::V, STEP = 4 * EV, NT = 4, U = 2;
+  constexpr int EV = El<T>::V, STEP = 4 * EV, NT = 4, U = RT == 1 ? 4 : 1;
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, n16 = lane & 15, g = lane >> 4;
-  const int h = blockIdx.z, c0 = blockIdx.y * 16 * NT;
-  const long t0 = ((long)blockIdx.x * 4 + wv) * 16 * RT;
-  if (t0 >= rows) return;
+  const int h = blockIdx.z, c0 = (blockIdx.y * (4 / WT) + wv / WT) * 16 * NT;
+  const long t0 = ((long)blockIdx.x * WT + wv % WT) * 16 * RT;
+  if (t0 >= rows || c0 >= N) return;   // no barrier in this kernel
   const T* xr[RT];
 #pragma unroll
   for (int r = 0; r < RT; ++r) xr[r] = x + min(t0 + 16 * r + n16, rows - 1) * xs + h * xh;
@@ -91,13 +91,12 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const T* __restrict__ 
 template <typename T>
 int head_linear_t(const void* x, long xs, long xh, const void* w, int H, int N, int K, long rows, void* out, long os, long oh, int vec, int vst,
                   hipStream_t st) {
-  const unsigned gy = (unsigned)((N + 63) / 64);
-  if (rows > 128)
-    head_linear_kernel<T, 2><<<dim3((unsigned)((rows + 127) / 128), gy, (unsigned)H), 256, 0, st>>>((const T*)x, xs, xh, (const T*)w, N, K, rows,
-                                                                                                  (T*)out, os, oh, vec, vst);
-  else
-    head_linear_kernel<T, 1><<<dim3((unsigned)((rows + 63) / 64), gy, (unsigned)H), 256, 0, st>>>((const T*)x, xs, xh, (const T*)w, N, K, rows,
-                                                                                                (T*)out, os, oh, vec, vst);
+#define LK_HEAD(RT, WT)                                                                                                                     \
+  head_linear_kernel<T, RT, WT><<<dim3((unsigned)((rows + 16 * RT * WT - 1) / (16 * RT * WT)), (unsigned)((N + 64 * (4 / WT) - 1) / (64 * (4 / WT))), \
+                                       (unsigned)H), 256, 0, st>>>((const T*)x, xs, xh, (const T*)w, N, K, rows, (T*)out, os, oh, vec, vst)
+  if (rows > 128) LK_HEAD(4, 2);
+  else LK_HEAD(1, 4);
+#undef LK_HEAD
   LK_CHECK_LAUNCH();
   return 0;
 }

@@ -346,7 +346,8 @@ int lk_router_choice(const void* h, long hs, const void* w, int E, int K, long r
 // csrc/mlstm.hip: matrix memory with exponential gates (S [slots, H, dk, dv], n | m [slots, H, ceil(dv / 64), dk + 4])
 int lk_mlstm_scan(const void* q, long qs, const void* k, long ks, const void* v, long vs, int esz, const float* gates, long gs, float q_scale,
                   float* S, float* nm, const int* cu, const int* slots, const int* positions, int seqs, int H, int dk, int dv, float* o,
-                  long os, int max_len, hipStream_t st);
+                  long os, int max_len, float* pre, hipStream_t st);
+int lk_mlstm_chunk_min();
 
 // csrc/head_linear.hip: out[t, h, :N] = w[h] x[t, h xh : h xh + K]
 int lk_head_linear(const void* x, long xs, long xh, const void* w, int H, int N, int K, long rows, void* out, long os, long oh, int esz,

@@ -13,8 +13,8 @@
 // LDS rows are unpadded; the 16-byte pieces of a row are XOR-swizzled inside groups of 8 so that both kinds of reads are free of
 // bank conflicts.
 //
-// Prompt portions: a workgroup (8 waves) owns 128 columns = the heads of a block x consecutive queries of one sequence, tiles
-// double-buffered.  Decode rows: a workgroup (4 waves) owns a sequence and a block of at most 16 heads, each wave walks its own
+// Prompt portions: a workgroup owns 128 columns = the heads of a block x consecutive queries of one sequence (16 or 32
+// columns per wave), tiles double-buffered.  Decode rows: a workgroup (4 waves) owns a sequence and a block of at most 16 heads, each wave walks its own
 // tiles (LDS-DMA into a wave-private region), merged through LDS; key splits over workgroups are merged by a second kernel.
 // f32 rows (and latents wider than the instances) run on a plain kernel, one workgroup per (row, head).
 //
@@ -52,59 +52,71 @@ LK_DEVICE int first_key(int qpos, int window) { return window > 0 ? max(0, qpos 
 
 LK_DEVICE int swz(int row) { return ((row & 3) << 1) | ((row >> 2) & 1); }
 
-// 32 staged rows (keys kb .. kb + 31) against this wave's 16 columns.  m: running maximum (base-2 scores; equal in the four lane
-// groups of a column), l: this lane group's share of the sum, o: O^T accumulators.  qpos < 0: column without a query.
-template <int RP, int RDP>
-LK_DEVICE void lat_tile(const bf16_t* tile, const uint4_t (&qf)[(RP + RDP) / 32], int kb, int qpos, int klo, float s2, float& m, float& l,
-                        floatx4 (&o)[RP / 16]) {
+// a column's running maximum moves only when a score exceeds it by this much (base 2): weights stay below 2^8, and the
+// accumulators are rescaled about once per column instead of at every new maximum
+constexpr float kMaxSlack = 8.f;
+
+// 32 staged rows (keys kb .. kb + 31) against CG groups of 16 columns: a row fragment read from LDS serves all groups.  m: running
+// maximum (base-2 scores; equal in the four lane groups of a column), l: this lane group's share of the sum, o: O^T
+// accumulators.  qpos < 0: column without a query.
+template <int RP, int RDP, int CG>
+LK_DEVICE void lat_tile(const bf16_t* tile, const uint4_t (&qf)[CG][(RP + RDP) / 32], int kb, const int (&qpos)[CG], const int (&klo)[CG], float s2,
+                        float (&m)[CG], float (&l)[CG], floatx4 (&o)[CG][RP / 16]) {
   constexpr int KD = RP + RDP, NKS = KD / 32, VT = RP / 16;
   const int lane = threadIdx.x & 63, n16 = lane & 15, g = lane >> 4;
   const unsigned char* base = reinterpret_cast<const unsigned char*>(tile);
-  floatx4 c[2];
+  floatx4 c[CG][2];
 #pragma unroll
   for (int t = 0; t < 2; ++t) {
-    c[t] = floatx4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int x = 0; x < CG; ++x) c[x][t] = floatx4{0.f, 0.f, 0.f, 0.f};
     const unsigned char* kr = base + (16 * t + n16) * KD * 2;
     const int sw = swz(n16), p0 = (g ^ sw) * 16, p1 = ((4 + g) ^ sw) * 16;
 #pragma unroll
     for (int s = 0; s < NKS; ++s) {
       const uint4_t a = *reinterpret_cast<const uint4_t*>(kr + (s >> 1) * 128 + ((s & 1) ? p1 : p0));
-      c[t] = mma_qk<bf16_t>(a, qf[s], c[t]);
+#pragma unroll
+      for (int x = 0; x < CG; ++x) c[x][t] = mma_qk<bf16_t>(a, qf[x][s], c[x][t]);
+      if (CG > 1 && s % 6 == 5) __builtin_amdgcn_sched_barrier(0);   // bounds how many fragments are in flight (registers)
     }
   }
-  float sc[2][4];
-  bool ok[2][4];
-  float mx = kNegBig;
+  short8 pb[CG];
 #pragma unroll
-  for (int t = 0; t < 2; ++t)
+  for (int x = 0; x < CG; ++x) {
+    float sc[2][4];
+    bool ok[2][4];
+    float mx = kNegBig;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int key = kb + 16 * t + 4 * g + j;
-      ok[t][j] = key <= qpos && key >= klo;
-      sc[t][j] = c[t][j] * s2;
-      if (ok[t][j]) mx = fmaxf(mx, sc[t][j]);
+    for (int t = 0; t < 2; ++t)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int key = kb + 16 * t + 4 * g + j;
+        ok[t][j] = key <= qpos[x] && key >= klo[x];
+        sc[t][j] = c[x][t][j] * s2;
+        if (ok[t][j]) mx = fmaxf(mx, sc[t][j]);
+      }
+    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    if (__any(mx > m[x] + kMaxSlack)) {
+      const float mn = fmaxf(m[x], mx), alpha = __builtin_amdgcn_exp2f(m[x] - mn);
+      m[x] = mn;
+      l[x] *= alpha;
+#pragma unroll
+      for (int vt = 0; vt < VT; ++vt) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) o[x][vt][j] *= alpha;
+        if (CG > 1 && vt % 4 == 3) __builtin_amdgcn_sched_barrier(0);
+      }
     }
-  mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-  mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-  const float mn = fmaxf(m, mx);
-  const float alpha = __builtin_amdgcn_exp2f(m - mn);
-  m = mn;
-  l *= alpha;
-  if (!__all(alpha == 1.f)) {
 #pragma unroll
-    for (int vt = 0; vt < VT; ++vt)
+    for (int t = 0; t < 2; ++t)
 #pragma unroll
-      for (int j = 0; j < 4; ++j) o[vt][j] *= alpha;
+      for (int j = 0; j < 4; ++j) {
+        const float p = ok[t][j] ? __builtin_amdgcn_exp2f(sc[t][j] - m[x]) : 0.f;
+        l[x] += p;
+        pb[x][4 * t + j] = (short)f2bf(p);
+      }
   }
-  short8 pb;
-#pragma unroll
-  for (int t = 0; t < 2; ++t)
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const float p = ok[t][j] ? __builtin_amdgcn_exp2f(sc[t][j] - mn) : 0.f;
-      l += p;
-      pb[4 * t + j] = (short)f2bf(p);
-    }
   const int qq = n16 >> 2, pp = n16 & 3, sw = swz(4 * g + qq);   // rows 4g + qq and 16 + 4g + qq have the same swizzle
   const unsigned char* vr = base + (4 * g + qq) * KD * 2 + 8 * (pp & 1);
   int voff[4];
@@ -116,7 +128,9 @@ LK_DEVICE void lat_tile(const bf16_t* tile, const uint4_t (&qf)[(RP + RDP) / 32]
     const short4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4_ptr)(a0));
     const short4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4_ptr)(a0 + 16 * KD * 2));
     const short8 a = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
-    o[vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb, o[vt], 0, 0, 0);
+#pragma unroll
+    for (int x = 0; x < CG; ++x) o[x][vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb[x], o[x][vt], 0, 0, 0);
+    if (CG > 1 && vt % 4 == 3) __builtin_amdgcn_sched_barrier(0);
   }
 }
 
@@ -134,26 +148,33 @@ LK_DEVICE long group_row(const int* bt, int BS, int kg, int last) {
   return (long)bt[k / BS] * BS + k % BS;
 }
 
-constexpr int kPreWaves = 8, kPreCols = 16 * kPreWaves;
+constexpr int kPreCols = 128;
+// column groups per wave: two where the accumulators of both fit the registers
+template <int RP>
+constexpr int pre_groups() { return RP <= 256 ? 2 : 1; }
+template <int RP>
+constexpr int pre_waves() { return kPreCols / (16 * pre_groups<RP>()); }
 
-// grid (query tiles, head blocks): tile x is found by walking the sequences (at most ceil(qlen / NQ) tiles each)
+// grid (query tiles, head blocks): tile x is found by walking the sequences (at most ceil(qlen / NQ) tiles each, a sequence's last
+// queries first: they see the most keys)
 template <int RP, int RDP>
-__global__ __launch_bounds__(kPreWaves * 64) void lat_prefill_kernel(LatParams p, const int* __restrict__ cu_q, const int* __restrict__ ctx_lens,
+__global__ __launch_bounds__(pre_waves<RP>() * 64) void lat_prefill_kernel(LatParams p, const int* __restrict__ cu_q, const int* __restrict__ ctx_lens,
                                                                      int nseq) {
-  constexpr int KD = RP + RDP, CPR = KD / 8, VT = RP / 16, NCH = 32 * CPR, NL = (NCH + kPreWaves * 64 - 1) / (kPreWaves * 64);
+  constexpr int KD = RP + RDP, CPR = KD / 8, VT = RP / 16, NCH = 32 * CPR, NT = pre_waves<RP>() * 64, NL = (NCH + NT - 1) / NT,
+                CG = pre_groups<RP>();
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   bf16_t* const buf = reinterpret_cast<bf16_t*>(smem);   // two tiles of 32 rows
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, n16 = lane & 15, g = lane >> 4;
   const int NQ = kPreCols / p.HC;
   int b = -1, q0 = 0;
   {
-    const int tile = xcd_remap(blockIdx.x, gridDim.x);
+    const int tile = blockIdx.x;
     int acc = 0;
     for (int i = 0; i < nseq; ++i) {
       const int nt = (cu_q[i + 1] - cu_q[i] + NQ - 1) / NQ;
       if (tile < acc + nt) {
         b = i;
-        q0 = (tile - acc) * NQ;
+        q0 = (nt - 1 - (tile - acc)) * NQ;
         break;
       }
       acc += nt;
@@ -161,22 +182,29 @@ __global__ __launch_bounds__(kPreWaves * 64) void lat_prefill_kernel(LatParams p
   }
   if (b < 0) return;   // the whole workgroup leaves
   const int qbeg = cu_q[b], qlen = cu_q[b + 1] - qbeg, ctx = ctx_lens[b], past = ctx - qlen;
-  const int c = 16 * w + n16, qi = q0 + c / p.HC, head = blockIdx.y * p.HC + c % p.HC;
-  const bool valid = c / p.HC < NQ && qi < qlen && head < p.H;
-  const int qpos = valid ? past + qi : -1, klo = first_key(qpos, p.window);
-  const bf16_t* qrow = reinterpret_cast<const bf16_t*>(p.q) + (long)(qbeg + min(qi, qlen - 1)) * p.qs + (long)min(head, p.H - 1) * KD;
-  uint4_t qf[KD / 32];
-  load_q<RP, RDP>(qrow, valid, qf);
-  floatx4 o[VT];
+  uint4_t qf[CG][KD / 32];
+  floatx4 o[CG][VT];
+  float m[CG], l[CG];
+  int qpos[CG], klo[CG], whi = -1, wlo = 0x7fffffff;
 #pragma unroll
-  for (int vt = 0; vt < VT; ++vt) o[vt] = floatx4{0.f, 0.f, 0.f, 0.f};
-  float m = p.sink && valid ? p.sink[head] * kLog2e : kNegBig, l = p.sink && valid && g == 0 ? 1.f : 0.f;
+  for (int x = 0; x < CG; ++x) {
+    const int c = 16 * (CG * w + x) + n16, qi = q0 + c / p.HC, head = blockIdx.y * p.HC + c % p.HC;
+    const bool valid = c / p.HC < NQ && qi < qlen && head < p.H;
+    qpos[x] = valid ? past + qi : -1;
+    klo[x] = first_key(qpos[x], p.window);
+    load_q<RP, RDP>(reinterpret_cast<const bf16_t*>(p.q) + (long)(qbeg + min(qi, qlen - 1)) * p.qs + (long)min(head, p.H - 1) * KD, valid, qf[x]);
+#pragma unroll
+    for (int vt = 0; vt < VT; ++vt) o[x][vt] = floatx4{0.f, 0.f, 0.f, 0.f};
+    m[x] = p.sink && valid ? p.sink[head] * kLog2e : kNegBig;
+    l[x] = p.sink && valid && g == 0 ? 1.f : 0.f;
+    whi = max(whi, qpos[x]);
+    wlo = min(wlo, valid ? klo[x] : 0x7fffffff);
+  }
   const float s2 = p.scale * kLog2e;
   const int k1 = min(ctx, past + q0 + NQ), k0 = first_key(past + q0, p.window) & ~31, last = (k1 - 1) & ~15;
   const int* bt = p.bt + (long)b * p.bt_stride;
   const bf16_t* cache = reinterpret_cast<const bf16_t*>(p.cache);
   // this wave's columns see keys wlo .. whi only
-  int whi = qpos, wlo = valid ? klo : 0x7fffffff;
 #pragma unroll
   for (int x = 1; x < 16; x <<= 1) {
     whi = max(whi, __shfl_xor(whi, x, 64));
@@ -187,21 +215,15 @@ __global__ __launch_bounds__(kPreWaves * 64) void lat_prefill_kernel(LatParams p
     const long r0 = group_row(bt, p.BS, kb, last), r1 = group_row(bt, p.BS, kb + 16, last);
 #pragma unroll
     for (int i = 0; i < NL; ++i) {
-      const int x = tid + kPreWaves * 64 * i;
-      if (NCH % (kPreWaves * 64) == 0 || x < NCH) {
-        const int r = x / CPR, cc = x % CPR;
-        st[i] = ld16(cache + ((r < 16 ? r0 : r1) + (r & 15)) * KD + cc * 8);
-      }
+      const int x = tid + NT * i, r = x / CPR, cc = x % CPR;
+      if (NCH % NT == 0 || x < NCH) st[i] = ld16(cache + ((r < 16 ? r0 : r1) + (r & 15)) * KD + cc * 8);
     }
   };
   auto stage = [&](bf16_t* dst) {
 #pragma unroll
     for (int i = 0; i < NL; ++i) {
-      const int x = tid + kPreWaves * 64 * i;
-      if (NCH % (kPreWaves * 64) == 0 || x < NCH) {
-        const int r = x / CPR, cc = x % CPR;
-        *reinterpret_cast<uint4_t*>(dst + r * KD + ((cc & ~7) | ((cc & 7) ^ swz(r))) * 8) = st[i];
-      }
+      const int x = tid + NT * i, r = x / CPR, cc = x % CPR;
+      if (NCH % NT == 0 || x < NCH) *reinterpret_cast<uint4_t*>(dst + r * KD + ((cc & ~7) | ((cc & 7) ^ swz(r))) * 8) = st[i];
     }
   };
   fetch(k0);
@@ -211,22 +233,26 @@ __global__ __launch_bounds__(kPreWaves * 64) void lat_prefill_kernel(LatParams p
   for (int kb = k0; kb < k1; kb += 32) {
     const bool more = kb + 32 < k1;
     if (more) fetch(kb + 32);
-    if (kb <= whi && kb + 31 >= wlo) lat_tile<RP, RDP>(buf + cur * 32 * KD, qf, kb, qpos, klo, s2, m, l, o);
+    if (kb <= whi && kb + 31 >= wlo) lat_tile<RP, RDP, CG>(buf + cur * 32 * KD, qf, kb, qpos, klo, s2, m, l, o);
     if (more) stage(buf + (cur ^ 1) * 32 * KD);
     __syncthreads();
     cur ^= 1;
   }
-  l += __shfl_xor(l, 16, 64);
-  l += __shfl_xor(l, 32, 64);
-  if (valid) {
-    const float f = l > 0.f ? 1.f / l : 0.f;
-    bf16_t* orow = reinterpret_cast<bf16_t*>(p.out) + (long)(qbeg + qi) * p.os + (long)head * RP + 4 * g;
 #pragma unroll
-    for (int vt = 0; vt < VT; ++vt) {
-      short4_t v;
+  for (int x = 0; x < CG; ++x) {
+    l[x] += __shfl_xor(l[x], 16, 64);
+    l[x] += __shfl_xor(l[x], 32, 64);
+    const int c = 16 * (CG * w + x) + n16, qi = q0 + c / p.HC, head = blockIdx.y * p.HC + c % p.HC;
+    if (qpos[x] >= 0) {
+      const float f = l[x] > 0.f ? 1.f / l[x] : 0.f;
+      bf16_t* orow = reinterpret_cast<bf16_t*>(p.out) + (long)(qbeg + qi) * p.os + (long)head * RP + 4 * g;
 #pragma unroll
-      for (int j = 0; j < 4; ++j) v[j] = (short)f2bf(o[vt][j] * f);
-      *reinterpret_cast<short4_t*>(orow + 16 * vt) = v;
+      for (int vt = 0; vt < VT; ++vt) {
+        short4_t v;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] = (short)f2bf(o[x][vt][j] * f);
+        *reinterpret_cast<short4_t*>(orow + 16 * vt) = v;
+      }
     }
   }
 }
@@ -241,42 +267,41 @@ __global__ __launch_bounds__(256) void lat_decode_kernel(LatParams p, const int*
   const int head = blockIdx.y * p.HC + n16;
   const bool valid = n16 < p.HC && head < p.H && ctx > 0;
   unsigned char* region = smem + w * 64 * KD;
-  const int qpos = valid ? ctx - 1 : -1;
+  const int qpos[1] = {valid ? ctx - 1 : -1}, klo[1] = {first_key(ctx - 1, p.window)}, k0 = klo[0];
   const bf16_t* qrow = reinterpret_cast<const bf16_t*>(p.q) + (long)b * p.qs + (long)min(head, p.H - 1) * KD;
-  uint4_t qf[KD / 32];
-  load_q<RP, RDP>(qrow, valid, qf);
-  floatx4 o[VT];
+  uint4_t qf[1][KD / 32];
+  load_q<RP, RDP>(qrow, valid, qf[0]);
+  floatx4 o[1][VT];
 #pragma unroll
-  for (int vt = 0; vt < VT; ++vt) o[vt] = floatx4{0.f, 0.f, 0.f, 0.f};
+  for (int vt = 0; vt < VT; ++vt) o[0][vt] = floatx4{0.f, 0.f, 0.f, 0.f};
   const bool own_sink = p.sink && valid && z == 0 && w == 0;
-  float m = own_sink ? p.sink[head] * kLog2e : kNegBig, l = own_sink && g == 0 ? 1.f : 0.f;
+  float m[1] = {own_sink ? p.sink[head] * kLog2e : kNegBig}, l[1] = {own_sink && g == 0 ? 1.f : 0.f};
   const float s2 = p.scale * kLog2e;
-  const int klo = first_key(ctx - 1, p.window), k0 = klo & ~31, last = (ctx - 1) & ~15;
   const int nsteps = ctx > 0 ? (ctx - k0 + 31) / 32 : 0, spz = (nsteps + Z - 1) / Z, e1 = min(nsteps, (z + 1) * spz);
   const int* bt = p.bt + (long)b * p.bt_stride;
   const bf16_t* cache = reinterpret_cast<const bf16_t*>(p.cache);
   for (int step = z * spz + w; step < e1; step += 4) {
     const int kb = k0 + 32 * step;
-    const long r0 = group_row(bt, p.BS, kb, last), r1 = group_row(bt, p.BS, kb + 16, last);
+    // tiles start at the first visible key (a window of 32 n keys is n tiles): lane x looks up the cache row of key kb + x % 32
+    const int key = min(kb + (lane & 31), ctx - 1), mine = bt[key / p.BS] * p.BS + key % p.BS;
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // the previous tile's LDS reads are done
 #pragma unroll
     for (int i = 0; i < NCH / 64; ++i) {
       // LDS piece x = 64 i + lane of the region is position x % CPR of row x / CPR: it holds the source piece swizzled back
       const int x = 64 * i + lane, r = x / CPR, pos = x % CPR, cc = (pos & ~7) | ((pos & 7) ^ swz(r));
-      __builtin_amdgcn_global_load_lds((gbl_void_ptr)(cache + ((r < 16 ? r0 : r1) + (r & 15)) * KD + cc * 8), (lds_void_ptr)(region + i * 1024), 16,
-                                       0, 0);
+      __builtin_amdgcn_global_load_lds((gbl_void_ptr)(cache + (long)__shfl(mine, r, 64) * KD + cc * 8), (lds_void_ptr)(region + i * 1024), 16, 0, 0);
     }
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    lat_tile<RP, RDP>(reinterpret_cast<const bf16_t*>(region), qf, kb, qpos, klo, s2, m, l, o);
+    lat_tile<RP, RDP, 1>(reinterpret_cast<const bf16_t*>(region), qf, kb, qpos, klo, s2, m, l, o);
   }
   // ---- merge the 4 waves: (m, l) behind every region's O block, then O relative to the common maximum
-  l += __shfl_xor(l, 16, 64);
-  l += __shfl_xor(l, 32, 64);
+  l[0] += __shfl_xor(l[0], 16, 64);
+  l[0] += __shfl_xor(l[0], 32, 64);
   asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
   float* ml = reinterpret_cast<float*>(region + 64 * RP);   // RP * 16 f32 of O come first; KD > RP leaves room behind them
   if (g == 0) {
-    ml[n16] = m;
-    ml[16 + n16] = l;
+    ml[n16] = m[0];
+    ml[16 + n16] = l[0];
   }
   __syncthreads();
   float M = kNegBig, L = 0.f;
@@ -287,10 +312,10 @@ __global__ __launch_bounds__(256) void lat_decode_kernel(LatParams p, const int*
     const float* q = reinterpret_cast<const float*>(smem + i * 64 * KD + 64 * RP);
     L += q[16 + n16] * __builtin_amdgcn_exp2f(q[n16] - M);
   }
-  const float f = __builtin_amdgcn_exp2f(m - M);
+  const float f = __builtin_amdgcn_exp2f(m[0] - M);
   floatx4* ob = reinterpret_cast<floatx4*>(region);
 #pragma unroll
-  for (int vt = 0; vt < VT; ++vt) ob[vt * 64 + lane] = floatx4{o[vt][0] * f, o[vt][1] * f, o[vt][2] * f, o[vt][3] * f};
+  for (int vt = 0; vt < VT; ++vt) ob[vt * 64 + lane] = floatx4{o[0][vt][0] * f, o[0][vt][1] * f, o[0][vt][2] * f, o[0][vt][3] * f};
   __syncthreads();
   const float inv = L > 0.f ? 1.f / L : 0.f;
 #pragma unroll
@@ -519,7 +544,7 @@ int launch_prefill(const LatParams& p, const int* cu_q, const int* ctx, int nseq
   const int NQ = kPreCols / p.HC;
   const long tiles = (rows + NQ - 1) / NQ + nseq;   // every sequence ends with at most one partial tile
   LK_SET_MAX_LDS((lat_prefill_kernel<RP, RDP>), lds);
-  lat_prefill_kernel<RP, RDP><<<dim3((unsigned)tiles, (unsigned)((p.H + p.HC - 1) / p.HC)), kPreWaves * 64, lds, st>>>(p, cu_q, ctx, nseq);
+  lat_prefill_kernel<RP, RDP><<<dim3((unsigned)tiles, (unsigned)((p.H + p.HC - 1) / p.HC)), pre_waves<RP>() * 64, lds, st>>>(p, cu_q, ctx, nseq);
   LK_CHECK_LAUNCH();
   return 0;
 }

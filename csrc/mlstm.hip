@@ -155,21 +155,76 @@ __global__ __launch_bounds__(256) void mlstm_step_kernel(MlstmParams a) {
 // ---- chunked matrix form (prompt portions): the recurrence unrolled over chunks of 16 tokens, products on true-f32 MFMAs
 // (bf16 rows: the q.k products on bf16 MFMAs, exact products either way), the state in the accumulators' layout from
 // chunk to chunk.  With F_t = f_1 + .. + f_t inside the chunk, S, n, m the state before it, a_s = i_s - F_s:
-//   m_t = F_t + max(m, max_{s<=t} a_s)
-//   D_ts = exp(F_t + a_s - m_t)  (s <= t),     e_t = exp(F_t + m - m_t)
+//   m_t = F_t + max(m, max_{s<=t} a_s),   c_t = F_t - m_t
+//   D_ts = exp(c_t + a_s)  (s <= t),     e_t = exp(c_t + m)
 //   num_t = e_t S^T q_t + sum_s D_ts (q_t.k_s) v_s,      nq_t = e_t n.q_t + sum_s D_ts (q_t.k_s)
 //   S' = e_L S + sum_s D_Ls k_s v_s^T,   n' = e_L n + sum_s D_Ls k_s,   m' = m_L
-// Tokens past the end of the last chunk get f = 0, i = -1e30: they neither decay nor feed the state.
+// Nothing of a_s, c_t, e_t depends on S: a kernel of one wave per (sequence, head) runs over the gates first and leaves
+// (a_t, c_t, c_t + m, m_t) per token, so the chain of the chunk kernel is S alone.
+constexpr int kChunk = 16;
+
+template <int N>
+LK_DEVICE float row_shr(float old, float v) {   // lane i of a row of 16 gets lane i - N (the first N lanes: old)
+  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(__builtin_bit_cast(int, old), __builtin_bit_cast(int, v), 0x110 + N, 0xf, 0xf, false));
+}
+
+LK_DEVICE float lane_of(float v, int l) { return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), l)); }
+
+// grid (sequence, head), one wave: 64 tokens = 4 chunks per round.  pre: [T, H] of 4 floats
+__global__ __launch_bounds__(64) void mlstm_gates_kernel(MlstmParams a, floatx4* __restrict__ pre) {
+  const int s = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+  const int row0 = a.cu[s], len = a.cu[s + 1] - row0, slot = a.slots[s];
+  if (len <= 0 || slot < 0) return;
+  float m = a.positions[row0] == 0 ? 0.f : a.nm[((long)slot * a.H + h) * a.Z * (a.dk + 4) + a.dk];
+  const float* gi = a.gates + (long)row0 * a.gs + h;
+  float ni = -1e30f, nf = 0.f;
+  if (lane < len) {
+    ni = gi[(long)lane * a.gs];
+    nf = gi[(long)lane * a.gs + a.H];
+  }
+  for (int t0 = 0; t0 < len; t0 += 64) {
+    const float ig = ni;
+    float F = nf;
+    const int tn = t0 + 64 + lane;
+    ni = -1e30f;
+    nf = 0.f;
+    if (tn < len) {   // the next round's gates travel under this round's scans
+      ni = gi[(long)tn * a.gs];
+      nf = gi[(long)tn * a.gs + a.H];
+    }
+    F += row_shr<1>(0.f, F);
+    F += row_shr<2>(0.f, F);
+    F += row_shr<4>(0.f, F);
+    F += row_shr<8>(0.f, F);
+    const float as = ig - F;
+    float am = as;
+    am = fmaxf(am, row_shr<1>(-1e30f, am));
+    am = fmaxf(am, row_shr<2>(-1e30f, am));
+    am = fmaxf(am, row_shr<4>(-1e30f, am));
+    am = fmaxf(am, row_shr<8>(-1e30f, am));
+    float min_ = m;
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      if ((lane >> 4) == c) min_ = m;
+      m = lane_of(F, 16 * c + 15) + fmaxf(m, lane_of(am, 16 * c + 15));
+    }
+    const float mt = F + fmaxf(min_, am);
+    if (t0 + lane < len) pre[(long)(row0 + t0 + lane) * a.H + h] = floatx4{as, F - mt, F - mt + min_, mt};
+  }
+}
+
 // grid (sequence, head, column block): wave w owns the 16 state columns j0 + 16 w .. + 15 (all dk rows: NR accumulator tiles).
+// Tokens past the end of the last chunk get a = -1e30 and the last token's c, m: they neither decay nor feed the state.
 template <typename T, int NR>
-__global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a) {
-  constexpr int NP = NR * 16, LD = NP + 4, L = 16, EV = 16 / sizeof(T), LH = NP + 8;
+__global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a, const floatx4* __restrict__ pre) {
+  constexpr int NP = NR * 16, LD = NP + 4, L = kChunk, EV = 16 / sizeof(T), LH = NP + 8;
   constexpr bool BF = sizeof(T) == 2 && NP % 32 == 0;
   __shared__ __attribute__((aligned(16))) float sk[L][LD];
   __shared__ __attribute__((aligned(16))) float sq[L][LD];
   __shared__ __attribute__((aligned(16))) bf16_t hk[BF ? L : 1][BF ? LH : 8];   // the raw bf16 rows (q.k products)
   __shared__ __attribute__((aligned(16))) bf16_t hq[BF ? L : 1][BF ? LH : 8];
-  __shared__ float sv[L][kColBlock], sn[2][NP], si[L], sf[L];
+  __shared__ __attribute__((aligned(16))) float sv[L][kColBlock + 4], sn[2][NP];
+  __shared__ __attribute__((aligned(16))) float ga[L], gc[L], ge[L], gw[L], gm[L];   // a_s, c_t, e_t, D_Ls, exp(-m_t)
   const int s = blockIdx.x, h = blockIdx.y, z = blockIdx.z, tid = threadIdx.x, j0 = z * kColBlock;
   const int lane = tid & 63, w = tid >> 6, n16 = lane & 15, g = lane >> 4;
   const int col = j0 + 16 * w + n16;
@@ -180,6 +235,10 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a) {
     zero_rows(a, row0, len, h, j0, 256);
     return;
   }
+  auto ex = [](float x) {   // accurate exponential for f32 rows, the hardware one for bf16 rows (whose own rounding is 2^-9)
+    if constexpr (sizeof(T) == 4) return expf(x);
+    else return __expf(x);
+  };
   const bool fresh = a.positions[row0] == 0;
   float* Sg = a.S + ((long)slot * a.H + h) * a.dk * a.dv + (cv ? col : 0);
   float* nmg = a.nm + (((long)slot * a.H + h) * a.Z + z) * (a.dk + 4);
@@ -191,7 +250,6 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a) {
       const int i = nt * 16 + 4 * g + j;
       S[nt][j] = (!fresh && cv && i < a.dk) ? Sg[(long)i * a.dv] : 0.f;
     }
-  float m = fresh ? 0.f : nmg[a.dk];
   for (int i = tid; i < NP; i += 256) sn[0][i] = (!fresh && i < a.dk) ? nmg[i] : 0.f;
   const T* qg = reinterpret_cast<const T*>(a.q) + (long)h * a.dk;
   const T* kg = reinterpret_cast<const T*>(a.k) + (long)h * a.dk;
@@ -200,28 +258,29 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a) {
                    (reinterpret_cast<uintptr_t>(kg) & 15) == 0;
   // the next chunk's operands are requested before this chunk's products are issued
   constexpr int CPR = NP / EV, NPF = (2 * L * CPR + 255) / 256;
-  uint4_t pre[NPF];
-  float prev_[4], prei = 0.f, pref = 0.f;
+  uint4_t stg[NPF];
+  float stv_[4];
+  floatx4 gt0 = {-1e30f, 0.f, 0.f, 0.f}, gl0 = {0.f, 0.f, 0.f, 0.f};   // this token's and the chunk's last token's gate terms
   auto fetch = [&](int t0) {
     const int tl = min(L, len - t0), ncpr = a.dk / EV;
 #pragma unroll
     for (int x = 0; x < NPF; ++x) {
       const int i = tid + 256 * x;
-      pre[x] = uint4_t{0u, 0u, 0u, 0u};
+      stg[x] = uint4_t{0u, 0u, 0u, 0u};
       if (i < 2 * L * CPR) {
         const int which = i / (L * CPR), r = i % (L * CPR), t = r / CPR, c = r % CPR;
         if (t < tl && c < ncpr)
-          pre[x] = *reinterpret_cast<const uint4_t*>((which ? qg + (long)(row0 + t0 + t) * a.qs : kg + (long)(row0 + t0 + t) * a.ks) + c * EV);
+          stg[x] = *reinterpret_cast<const uint4_t*>((which ? qg + (long)(row0 + t0 + t) * a.qs : kg + (long)(row0 + t0 + t) * a.ks) + c * EV);
       }
     }
 #pragma unroll
     for (int x = 0; x < 4; ++x) {
       const int i = tid + 256 * x, t = i >> 6, c = i & 63;
-      prev_[x] = (t < tl && j0 + c < a.dv) ? ldf<T>(vg + (long)(row0 + t0 + t) * a.vs + j0 + c) : 0.f;
+      stv_[x] = (t < tl && j0 + c < a.dv) ? ldf<T>(vg + (long)(row0 + t0 + t) * a.vs + j0 + c) : 0.f;
     }
     if (tid < L) {
-      prei = tid < tl ? a.gates[(long)(row0 + t0 + tid) * a.gs + h] : -1e30f;
-      pref = tid < tl ? a.gates[(long)(row0 + t0 + tid) * a.gs + a.H + h] : 0.f;
+      gl0 = pre[(long)(row0 + t0 + tl - 1) * a.H + h];
+      gt0 = tid < tl ? pre[(long)(row0 + t0 + tid) * a.H + h] : floatx4{-1e30f, gl0[1], gl0[2], gl0[3]};
     }
   };
   fetch(0);
@@ -236,15 +295,14 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a) {
         if (i < 2 * L * CPR) {
           const int which = i / (L * CPR), r = i % (L * CPR), t = r / CPR, c = r % CPR;
           float* dst = (which ? sq[t] : sk[t]) + c * EV;
+          const float f = which ? a.q_scale : 1.f;
           if constexpr (sizeof(T) == 2) {
-            const short8 v = __builtin_bit_cast(short8, pre[x]);
-            const float f = which ? a.q_scale : 1.f;
+            const short8 v = __builtin_bit_cast(short8, stg[x]);
             *reinterpret_cast<floatx4*>(dst) = floatx4{bf2f((bf16_t)v[0]) * f, bf2f((bf16_t)v[1]) * f, bf2f((bf16_t)v[2]) * f, bf2f((bf16_t)v[3]) * f};
             *reinterpret_cast<floatx4*>(dst + 4) = floatx4{bf2f((bf16_t)v[4]) * f, bf2f((bf16_t)v[5]) * f, bf2f((bf16_t)v[6]) * f, bf2f((bf16_t)v[7]) * f};
-            if constexpr (BF) *reinterpret_cast<uint4_t*>((which ? hq[t] : hk[t]) + c * EV) = pre[x];
+            if constexpr (BF) *reinterpret_cast<uint4_t*>((which ? hq[t] : hk[t]) + c * EV) = stg[x];
           } else {
-            const floatx4 v = __builtin_bit_cast(floatx4, pre[x]);
-            const float f = which ? a.q_scale : 1.f;
+            const floatx4 v = __builtin_bit_cast(floatx4, stg[x]);
             *reinterpret_cast<floatx4*>(dst) = floatx4{v[0] * f, v[1] * f, v[2] * f, v[3] * f};
           }
         }
@@ -263,31 +321,17 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a) {
 #pragma unroll
     for (int x = 0; x < 4; ++x) {
       const int i = tid + 256 * x;
-      sv[i >> 6][i & 63] = prev_[x];
+      sv[i >> 6][i & 63] = stv_[x];
     }
     if (tid < L) {
-      si[tid] = prei;
-      sf[tid] = pref;
+      ga[tid] = gt0[0];
+      gc[tid] = gt0[1];
+      ge[tid] = ex(gt0[2]);
+      gm[tid] = ex(-gt0[3]);
+      gw[tid] = ex(gl0[1] + gt0[0]);
     }
     __syncthreads();
     if (t0 + L < len) fetch(t0 + L);
-    // inside every 16-lane group: lane t ends up with F_t and max_{s<=t} a_s
-    float F = sf[n16];
-#pragma unroll
-    for (int o = 1; o < 16; o <<= 1) {
-      const float v = __shfl_up(F, o, 16);
-      if (n16 >= o) F += v;
-    }
-    const float as = si[n16] - F;
-    float am = as;
-#pragma unroll
-    for (int o = 1; o < 16; o <<= 1) {
-      const float v = __shfl_up(am, o, 16);
-      if (n16 >= o) am = fmaxf(am, v);
-    }
-    const float mt = F + fmaxf(m, am);          // m_t of t = n16
-    const float et = expf(F + m - mt);
-    const float Fl = __shfl(F, 15, 16), ml = __shfl(mt, 15, 16);
     // G^T: lane (t = n16, g) gets G[t][s = 4g + j] = q_t . k_s
     floatx4 gt = {0.f, 0.f, 0.f, 0.f};
     if constexpr (BF) {
@@ -308,16 +352,6 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a) {
         for (int j = 0; j < 4; ++j) gt = __builtin_amdgcn_mfma_f32_16x16x4f32(a4[j], b4[j], gt, 0, 0, 0);
       }
     }
-    float M[4], xv[4], wl[4], ms = 0.f;
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int sj = 4 * g + j;
-      const float a_s = __shfl(as, sj, 16);
-      M[j] = sj <= n16 ? gt[j] * expf(F + a_s - mt) : 0.f;
-      ms += M[j];
-      xv[j] = sv[sj][16 * w + n16];
-      wl[j] = expf(Fl + a_s - ml);
-    }
     // num: rows t = 4g + j, column n16 of this wave's tile; n . q of t = n16 beside it
     floatx4 ya = {0.f, 0.f, 0.f, 0.f};
     float nq = 0.f;
@@ -331,13 +365,22 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a) {
         nq += q4[j] * n4[j];
       }
     }
-    nq = et * nq + ms;   // e_t is the same in the four lane groups of t
-    // (each group holds its quarter of both sums: e_t distributes over them)
+    const floatx4 a4 = *reinterpret_cast<const floatx4*>(&ga[4 * g]), e4 = *reinterpret_cast<const floatx4*>(&ge[4 * g]),
+                  w4 = *reinterpret_cast<const floatx4*>(&gw[4 * g]);
+    const float ct = gc[n16];
+    float M[4], xv[4];
+    nq *= ge[n16];   // (each lane group holds its quarter of both sums of t = n16)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      M[j] = 4 * g + j <= n16 ? gt[j] * ex(ct + a4[j]) : 0.f;
+      nq += M[j];
+      xv[j] = sv[4 * g + j][16 * w + n16];
+    }
     nq += __shfl_xor(nq, 16, 64);
     nq += __shfl_xor(nq, 32, 64);
-    const float rden = 1.f / (fmaxf(fabsf(nq), expf(-mt)) + kDenEps);
+    const float rden = 1.f / (fmaxf(fabsf(nq), gm[n16]) + kDenEps);
 #pragma unroll
-    for (int j = 0; j < 4; ++j) ya[j] *= __shfl(et, 4 * g + j, 16);
+    for (int j = 0; j < 4; ++j) ya[j] *= e4[j];
 #pragma unroll
     for (int j = 0; j < 4; ++j) ya = __builtin_amdgcn_mfma_f32_16x16x4f32(M[j], xv[j], ya, 0, 0, 0);
 #pragma unroll
@@ -347,26 +390,30 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a) {
       if (cv && t < tl) a.o[(long)(row0 + t0 + t) * a.os + (long)h * a.dv + col] = ya[j] * rd;
     }
     // state: rows i = 16 nt + 4g + j, column n16
-    const float dec = expf(Fl + m - ml);
+    const float dec = ge[L - 1];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) xv[j] *= w4[j];   // D_Ls v_s
 #pragma unroll
     for (int nt = 0; nt < NR; ++nt) {
 #pragma unroll
       for (int j = 0; j < 4; ++j) S[nt][j] *= dec;
-#pragma unroll
-      for (int j = 0; j < 4; ++j)
-        S[nt] = __builtin_amdgcn_mfma_f32_16x16x4f32(sk[4 * g + j][nt * 16 + n16] * wl[j], xv[j], S[nt], 0, 0, 0);
     }
-    float ws[L];         // D_Ls of every s, uniform
 #pragma unroll
-    for (int x = 0; x < L; ++x) ws[x] = __shfl(wl[x & 3], 16 * (x >> 2), 64);
-    for (int i = tid; i < NP; i += 256) {
-      float v = dec * sn[cur][i];
+    for (int j = 0; j < 4; ++j)
 #pragma unroll
-      for (int x = 0; x < L; ++x) v += ws[x] * sk[x][i];
-      sn[cur ^ 1][i] = v;
+      for (int nt = 0; nt < NR; ++nt) S[nt] = __builtin_amdgcn_mfma_f32_16x16x4f32(sk[4 * g + j][nt * 16 + n16], xv[j], S[nt], 0, 0, 0);
+    // n: a wave owns NP / 4 of its entries, PARTS lanes share one and take 16 / PARTS tokens each
+    constexpr int NW = NP / 4, PARTS = 64 / NW;
+    {
+      const int i = w * NW + lane % NW, part = lane / NW;
+      float v = 0.f;
+#pragma unroll
+      for (int x = 0; x < L / PARTS; ++x) v += gw[part * (L / PARTS) + x] * sk[part * (L / PARTS) + x][i];
+#pragma unroll
+      for (int d = NW; d < 64; d <<= 1) v += __shfl_xor(v, d, 64);
+      if (part == 0) sn[cur ^ 1][i] = dec * sn[cur][i] + v;
     }
     cur ^= 1;
-    m = ml;
   }
   __syncthreads();
   if (cv) {
@@ -379,14 +426,17 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a) {
       }
   }
   for (int i = tid; i < a.dk; i += 256) nmg[i] = sn[cur][i];
-  if (tid == 0) nmg[a.dk] = m;
+  if (tid == 0) nmg[a.dk] = pre[(long)(row0 + len - 1) * a.H + h][3];
 }
 
 template <typename T>
-int scan_t(const MlstmParams& a, int S, int max_len, hipStream_t st) {
+int scan_t(const MlstmParams& a, int S, int max_len, floatx4* pre, hipStream_t st) {
   const dim3 grid((unsigned)S, (unsigned)a.H, (unsigned)a.Z);
   if (max_len >= kChunkMin) {
-#define LK_CHUNK(NR) mlstm_chunk_kernel<T, NR><<<grid, 256, 0, st>>>(a)
+    if (!pre) return -1;
+    mlstm_gates_kernel<<<dim3((unsigned)S, (unsigned)a.H), 64, 0, st>>>(a, pre);
+    LK_CHECK_LAUNCH();
+#define LK_CHUNK(NR) mlstm_chunk_kernel<T, NR><<<grid, 256, 0, st>>>(a, pre)
     if (a.dk <= 16) LK_CHUNK(1);
     else if (a.dk <= 32) LK_CHUNK(2);
     else if (a.dk <= 64) LK_CHUNK(4);
@@ -413,14 +463,18 @@ int scan_t(const MlstmParams& a, int S, int max_len, hipStream_t st) {
 
 }  // namespace
 
+// the chunked form runs when some sequence of the step has this many rows: it needs `pre`, [rows, H, 4] f32 scratch
+int lk_mlstm_chunk_min() { return kChunkMin; }
+
 int lk_mlstm_scan(const void* q, long qs, const void* k, long ks, const void* v, long vs, int esz, const float* gates, long gs, float q_scale,
                   float* S, float* nm, const int* cu, const int* slots, const int* positions, int seqs, int H, int dk, int dv, float* o,
-                  long os, int max_len, hipStream_t st) {
+                  long os, int max_len, float* pre, hipStream_t st) {
   if (seqs <= 0) return 0;
   if (H < 1 || H > 65535 || dk < 1 || dk > 256 || dv < 1 || (dv + kColBlock - 1) / kColBlock > 65535) return -1;
   MlstmParams a;
   a.q = q; a.k = k; a.v = v; a.qs = qs; a.ks = ks; a.vs = vs; a.gates = gates; a.gs = gs; a.q_scale = q_scale; a.S = S; a.nm = nm;
   a.cu = cu; a.slots = slots; a.positions = positions; a.o = o; a.os = os; a.H = H; a.dk = dk; a.dv = dv;
   a.Z = (dv + kColBlock - 1) / kColBlock;
-  return esz == 2 ? scan_t<bf16_t>(a, seqs, max_len, st) : scan_t<float>(a, seqs, max_len, st);
+  return esz == 2 ? scan_t<bf16_t>(a, seqs, max_len, reinterpret_cast<floatx4*>(pre), st)
+                  : scan_t<float>(a, seqs, max_len, reinterpret_cast<floatx4*>(pre), st);
 }

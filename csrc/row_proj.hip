@@ -132,8 +132,9 @@ __global__ __launch_bounds__(kWaves * 64) void router_choice_kernel(const T* __r
                                                                     int* __restrict__ experts, float* __restrict__ weights) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   float* red = lds;
-  float* zs = lds + kWaves * kRowTile * kCols;
+  float* zs = lds + max(kWaves * kRowTile * kCols, 2 * kWaves * E);
   project<T>(h, hs, w, E, K, rows, vec, red, zs, E);
+  double* sc = reinterpret_cast<double*>(lds) + (long)(threadIdx.x >> 6) * E;   // this wave's scores: the partial sums have been consumed
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, per = E / groups;
   const double ninf = -__builtin_huge_val();
   for (int r = wv; r < kRowTile; r += kWaves) {
@@ -143,27 +144,34 @@ __global__ __launch_bounds__(kWaves * 64) void router_choice_kernel(const T* __r
     float zm = -__builtin_huge_valf();
     for (int e = lane; e < E; e += 64) zm = fmaxf(zm, z[e]);
     zm = wave_max(zm);
-    double den = 0.0;
-    if (score == 1) {
-      for (int e = lane; e < E; e += 64) den += exp((double)z[e] - (double)zm);
-      den = wave_sum_d(den);
-    }
-    auto score_of = [&](int e) -> double {
-      return score == 1 ? exp((double)z[e] - (double)zm) / den : 1.0 / (1.0 + exp(-(double)z[e]));
-    };
-    double c[EPL];
+    // every lane evaluates its experts' scores once; LDS publishes them to the group scores and the choice
+    double c[EPL], den = 0.0;
 #pragma unroll
     for (int i = 0; i < EPL; ++i) {
       const int e = lane + 64 * i;
-      c[i] = e < E ? score_of(e) + (corr ? (double)corr[e] : 0.0) : ninf;
+      c[i] = e < E ? (score == 1 ? exp((double)z[e] - (double)zm) : 1.0 / (1.0 + exp(-(double)z[e]))) : 0.0;
+      den += c[i];
     }
+    const double inv = score == 1 ? 1.0 / wave_sum_d(den) : 1.0;
+#pragma unroll
+    for (int i = 0; i < EPL; ++i) {
+      const int e = lane + 64 * i;
+      if (e < E) {
+        c[i] *= inv;
+        sc[e] = c[i];
+        c[i] += corr ? (double)corr[e] : 0.0;
+      } else {
+        c[i] = ninf;
+      }
+    }
+    __builtin_amdgcn_wave_barrier();
     if (groups > 1) {   // at most 64 groups (host check): lane x holds group x's score
       double mine = ninf;
       if (lane < groups) {
         double b1 = ninf, b2 = ninf;
         for (int j = 0; j < per; ++j) {
           const int e = lane * per + j;
-          const double v = score_of(e) + (corr ? (double)corr[e] : 0.0);
+          const double v = sc[e] + (corr ? (double)corr[e] : 0.0);
           if (v > b1) { b2 = b1; b1 = v; } else if (v > b2) { b2 = v; }
         }
         mine = gscore == 1 ? b1 : b1 + (per > 1 ? b2 : 0.0);
@@ -195,7 +203,7 @@ __global__ __launch_bounds__(kWaves * 64) void router_choice_kernel(const T* __r
 #pragma unroll
       for (int i = 0; i < EPL; ++i)
         if (bi == lane + 64 * i) c[i] = ninf;
-      const double s = score_of(bi);
+      const double s = sc[bi];
       if (lane == k) { chosen_s = s; chosen_e = bi; }
       sum += s;
     }
@@ -225,7 +233,8 @@ int gate_t(const void* h, long hs, const void* w, const float* bias, int N, int 
 template <typename T, int EPL>
 int router_e(const void* h, long hs, const void* w, int E, int K, long rows, int top, int groups, int keep, float scale, int score,
              const float* corr, int gscore, int vec, int* experts, float* weights, hipStream_t st) {
-  const size_t lds = sizeof(float) * (kWaves * kRowTile * kCols + (size_t)kRowTile * E);
+  const size_t lds = sizeof(float) * ((size_t)(kWaves * kRowTile * kCols > 2 * kWaves * E ? kWaves * kRowTile * kCols : 2 * kWaves * E) +
+                                      (size_t)kRowTile * E);
   if (lds > 128 * 1024) return -1;
   LK_SET_MAX_LDS((router_choice_kernel<T, EPL>), 128 * 1024);
   router_choice_kernel<T, EPL><<<(unsigned)((rows + kRowTile - 1) / kRowTile), kWaves * 64, lds, st>>>(

@@ -16,7 +16,7 @@ import torch
 from ._ext import lib, use_hip
 
 __all__ = ["latent_row", "latent_prep", "latent_query_rot", "head_linear", "latent_attention_prefill", "latent_attention_decode",
-           "latent_decode_splits", "latent_heads_per_tile"]
+           "latent_decode_splits"]
 
 
 def latent_row(kv_rank: int, rot_dim: int) -> tuple:
@@ -87,15 +87,10 @@ def head_linear(x, w, x_head: int, out):
     return out
 
 
-def latent_heads_per_tile(H: int) -> int:
-    """Query heads a tile of 16 columns holds: the heads are dealt evenly over ceil(H / 16) blocks."""
-    return -(-H // -(-H // 16))
-
-
 def latent_decode_splits(B: int, H: int, span: int) -> int:
     """Workgroups per (sequence, head block) of the decode kernel: about one workgroup per CU, never more than one per 128 keys."""
     blocks = max(1, B * -(-H // 16))
-    return int(max(1, min(256 // blocks if blocks <= 256 else 1, -(-(span + 31) // 128))))
+    return int(max(1, min(256 // blocks if blocks <= 256 else 1, -(-span // 128))))
 
 
 def _rows(qa, kv, qpos, window: int, scale: float, sink, rp: int):
