@@ -215,7 +215,8 @@ __global__ __launch_bounds__(64) void mlstm_gates_kernel(MlstmParams a, floatx4*
 
 // grid (sequence, head, column block): wave w owns the 16 state columns j0 + 16 w .. + 15 (all dk rows: NR accumulator tiles).
 // Tokens past the end of the last chunk get a = -1e30 and the last token's c, m: they neither decay nor feed the state.
-template <typename T, int NR>
+// VEC: 16-byte pieces of q and k rows, 4 adjacent columns of v (host check).
+template <typename T, int NR, bool VEC>
 __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a, const floatx4* __restrict__ pre) {
   constexpr int NP = NR * 16, LD = NP + 4, L = kChunk, EV = 16 / sizeof(T), LH = NP + 8;
   constexpr bool BF = sizeof(T) == 2 && NP % 32 == 0;
@@ -244,51 +245,56 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a, const f
   float* nmg = a.nm + (((long)slot * a.H + h) * a.Z + z) * (a.dk + 4);
   floatx4 S[NR];
 #pragma unroll
-  for (int nt = 0; nt < NR; ++nt)
+  for (int nt = 0; nt < NR; ++nt) S[nt] = floatx4{0.f, 0.f, 0.f, 0.f};
+  if (!fresh) {   // (loads from clamped places, selected afterwards: all in flight together)
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int i = nt * 16 + 4 * g + j;
-      S[nt][j] = (!fresh && cv && i < a.dk) ? Sg[(long)i * a.dv] : 0.f;
-    }
+    for (int nt = 0; nt < NR; ++nt)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) S[nt][j] = Sg[(long)min(nt * 16 + 4 * g + j, a.dk - 1) * a.dv];
+#pragma unroll
+    for (int nt = 0; nt < NR; ++nt)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) S[nt][j] = cv && nt * 16 + 4 * g + j < a.dk ? S[nt][j] : 0.f;
+  }
   for (int i = tid; i < NP; i += 256) sn[0][i] = (!fresh && i < a.dk) ? nmg[i] : 0.f;
   const T* qg = reinterpret_cast<const T*>(a.q) + (long)h * a.dk;
   const T* kg = reinterpret_cast<const T*>(a.k) + (long)h * a.dk;
   const T* vg = reinterpret_cast<const T*>(a.v) + (long)h * a.dv;
-  const bool vec = a.dk % EV == 0 && a.qs % EV == 0 && a.ks % EV == 0 && (reinterpret_cast<uintptr_t>(qg) & 15) == 0 &&
-                   (reinterpret_cast<uintptr_t>(kg) & 15) == 0;
-  // the next chunk's operands are requested before this chunk's products are issued
+  // The next chunk's operands are requested before this chunk's products are issued, as raw pieces from clamped places: nothing
+  // is converted, masked or branched on until they are staged, so no load is waited for here.
   constexpr int CPR = NP / EV, NPF = (2 * L * CPR + 255) / 256;
+  const int vt = tid >> 4, vc = j0 + 4 * (tid & 15);   // this thread's token and first of 4 columns of v
   uint4_t stg[NPF];
-  float stv_[4];
-  floatx4 gt0 = {-1e30f, 0.f, 0.f, 0.f}, gl0 = {0.f, 0.f, 0.f, 0.f};   // this token's and the chunk's last token's gate terms
+  T stv[4];
+  floatx4 gt0, gl0;   // this token's and the chunk's last token's gate terms
   auto fetch = [&](int t0) {
     const int tl = min(L, len - t0), ncpr = a.dk / EV;
+    if constexpr (VEC) {
 #pragma unroll
-    for (int x = 0; x < NPF; ++x) {
-      const int i = tid + 256 * x;
-      stg[x] = uint4_t{0u, 0u, 0u, 0u};
-      if (i < 2 * L * CPR) {
-        const int which = i / (L * CPR), r = i % (L * CPR), t = r / CPR, c = r % CPR;
-        if (t < tl && c < ncpr)
-          stg[x] = *reinterpret_cast<const uint4_t*>((which ? qg + (long)(row0 + t0 + t) * a.qs : kg + (long)(row0 + t0 + t) * a.ks) + c * EV);
+      for (int x = 0; x < NPF; ++x) {
+        const int i = min(tid + 256 * x, 2 * L * CPR - 1);
+        const int which = i / (L * CPR), r = i % (L * CPR), t = min(r / CPR, tl - 1), c = min(r % CPR, ncpr - 1);
+        const T* src = which ? qg : kg;
+        stg[x] = *reinterpret_cast<const uint4_t*>(src + (long)(row0 + t0 + t) * (which ? a.qs : a.ks) + c * EV);
       }
     }
+    const T* vr = vg + (long)(row0 + t0 + min(vt, tl - 1)) * a.vs;
+    if constexpr (VEC) {
+      if constexpr (sizeof(T) == 2) *reinterpret_cast<short4_t*>(stv) = *reinterpret_cast<const short4_t*>(vr + min(vc, a.dv - 4));
+      else *reinterpret_cast<floatx4*>(stv) = *reinterpret_cast<const floatx4*>(vr + min(vc, a.dv - 4));
+    } else {
 #pragma unroll
-    for (int x = 0; x < 4; ++x) {
-      const int i = tid + 256 * x, t = i >> 6, c = i & 63;
-      stv_[x] = (t < tl && j0 + c < a.dv) ? ldf<T>(vg + (long)(row0 + t0 + t) * a.vs + j0 + c) : 0.f;
+      for (int e = 0; e < 4; ++e) stv[e] = vr[min(vc + e, a.dv - 1)];
     }
-    if (tid < L) {
-      gl0 = pre[(long)(row0 + t0 + tl - 1) * a.H + h];
-      gt0 = tid < tl ? pre[(long)(row0 + t0 + tid) * a.H + h] : floatx4{-1e30f, gl0[1], gl0[2], gl0[3]};
-    }
+    gl0 = pre[(long)(row0 + t0 + tl - 1) * a.H + h];
+    gt0 = pre[(long)(row0 + t0 + min(n16, tl - 1)) * a.H + h];
   };
   fetch(0);
   int cur = 0;
   for (int t0 = 0; t0 < len; t0 += L) {
     const int tl = min(L, len - t0);
     __syncthreads();   // the previous chunk has been consumed
-    if (vec) {
+    if constexpr (VEC) {
 #pragma unroll
       for (int x = 0; x < NPF; ++x) {
         const int i = tid + 256 * x;
@@ -296,6 +302,7 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a, const f
           const int which = i / (L * CPR), r = i % (L * CPR), t = r / CPR, c = r % CPR;
           float* dst = (which ? sq[t] : sk[t]) + c * EV;
           const float f = which ? a.q_scale : 1.f;
+          if (t >= tl || c >= a.dk / EV) stg[x] = uint4_t{0u, 0u, 0u, 0u};
           if constexpr (sizeof(T) == 2) {
             const short8 v = __builtin_bit_cast(short8, stg[x]);
             *reinterpret_cast<floatx4*>(dst) = floatx4{bf2f((bf16_t)v[0]) * f, bf2f((bf16_t)v[1]) * f, bf2f((bf16_t)v[2]) * f, bf2f((bf16_t)v[3]) * f};
@@ -318,17 +325,23 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmParams a, const f
         if constexpr (BF) (which ? hq[t] : hk[t])[c] = raw;
       }
     }
+    {
+      floatx4 v;
 #pragma unroll
-    for (int x = 0; x < 4; ++x) {
-      const int i = tid + 256 * x;
-      sv[i >> 6][i & 63] = stv_[x];
+      for (int e = 0; e < 4; ++e) v[e] = vt < tl && vc + e < a.dv ? ldf<T>(stv + e) : 0.f;
+      *reinterpret_cast<floatx4*>(&sv[vt][vc - j0]) = v;
     }
-    if (tid < L) {
-      ga[tid] = gt0[0];
-      gc[tid] = gt0[1];
-      ge[tid] = ex(gt0[2]);
-      gm[tid] = ex(-gt0[3]);
-      gw[tid] = ex(gl0[1] + gt0[0]);
+    {   // (every thread evaluates its token's terms, 16 of them store: no load is left in flight on a path that skips its use)
+      const bool in = n16 < tl;
+      const float as = in ? gt0[0] : -1e30f, cc = in ? gt0[1] : gl0[1], ee = ex(in ? gt0[2] : gl0[2]), mm = ex(in ? -gt0[3] : -gl0[3]),
+                  ww = ex(gl0[1] + as);
+      if (tid < L) {
+        ga[tid] = as;
+        gc[tid] = cc;
+        ge[tid] = ee;
+        gm[tid] = mm;
+        gw[tid] = ww;
+      }
     }
     __syncthreads();
     if (t0 + L < len) fetch(t0 + L);
@@ -436,12 +449,18 @@ int scan_t(const MlstmParams& a, int S, int max_len, floatx4* pre, hipStream_t s
     if (!pre) return -1;
     mlstm_gates_kernel<<<dim3((unsigned)S, (unsigned)a.H), 64, 0, st>>>(a, pre);
     LK_CHECK_LAUNCH();
-#define LK_CHUNK(NR) mlstm_chunk_kernel<T, NR><<<grid, 256, 0, st>>>(a, pre)
-    if (a.dk <= 16) LK_CHUNK(1);
-    else if (a.dk <= 32) LK_CHUNK(2);
-    else if (a.dk <= 64) LK_CHUNK(4);
-    else if (a.dk <= 128) LK_CHUNK(8);
-    else if (a.dk <= 256) LK_CHUNK(16);
+    constexpr int ev = 16 / (int)sizeof(T);
+    const auto al = [](const void* x, int b) { return reinterpret_cast<uintptr_t>(x) % b == 0; };
+    const bool cvec = a.dk % ev == 0 && a.qs % ev == 0 && a.ks % ev == 0 && al(a.q, 16) && al(a.k, 16) && a.dv % 4 == 0 && a.vs % 4 == 0 &&
+                      al(a.v, 4 * sizeof(T));
+#define LK_CHUNK(NR)                                                         \
+  if (cvec) mlstm_chunk_kernel<T, NR, true><<<grid, 256, 0, st>>>(a, pre);    \
+  else mlstm_chunk_kernel<T, NR, false><<<grid, 256, 0, st>>>(a, pre)
+    if (a.dk <= 16) { LK_CHUNK(1); }
+    else if (a.dk <= 32) { LK_CHUNK(2); }
+    else if (a.dk <= 64) { LK_CHUNK(4); }
+    else if (a.dk <= 128) { LK_CHUNK(8); }
+    else if (a.dk <= 256) { LK_CHUNK(16); }
     else return -1;
 #undef LK_CHUNK
   } else {
