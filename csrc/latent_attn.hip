@@ -10,10 +10,10 @@
 //   S^T (keys x columns) = rows . qa^T  on v_mfma_f32_16x16x32_bf16 (rows as 16-byte LDS fragments, queries in registers),
 //   O^T (latent x columns) += c^T . P^T with c^T by transposed LDS reads (ds_read_b64_tr_b16) and P^T straight from the S^T
 //   accumulators (both sides use the key order 4g + j, 16 + 4g + j).
-// LDS rows are unpadded; the 16-byte pieces of a row are XOR-swizzled inside groups of 8 so that both kinds of reads are free of
-// bank conflicts.
+// LDS rows are unpadded multiples of 128 bytes; the 16-byte pieces of a row are XOR-swizzled inside groups of 8 so that both kinds
+// of reads spread over the banks.
 //
-// Prompt portions: a workgroup owns 128 columns = the heads of a block x consecutive queries of one sequence (16 or 32
+// Prompt portions: a workgroup owns 128 columns = the heads of a block x consecutive queries of one sequence (32
 // columns per wave), tiles double-buffered.  Decode rows: a workgroup (4 waves) owns a sequence and a block of at most 16 heads, each wave walks its own
 // tiles (LDS-DMA into a wave-private region), merged through LDS; key splits over workgroups are merged by a second kernel.
 // f32 rows (and latents wider than the instances) run on a plain kernel, one workgroup per (row, head).
@@ -21,13 +21,14 @@
 // Masks are taken from absolute positions: a prompt cut anywhere, a decode row and a whole prompt are the same sums.
 //
 // lk_latent_prep / lk_latent_query_rot prepare the operands (norms, rotation in halves, the cache row) in f32.
+#include <type_traits>
+
 #include "common.h"
 #include "kernels.h"
 #include "attn_frag.h"
 
 namespace {
 
-typedef short4_t __attribute__((address_space(3))) * lds_s4_ptr;
 typedef __attribute__((address_space(3))) void* lds_void_ptr;
 typedef const __attribute__((address_space(1))) void* gbl_void_ptr;
 
@@ -50,36 +51,93 @@ struct LatParams {
 
 LK_DEVICE int first_key(int qpos, int window) { return window > 0 ? max(0, qpos - window + 1) : 0; }
 
-LK_DEVICE int swz(int row) { return ((row & 3) << 1) | ((row >> 2) & 1); }
+LK_DEVICE int swz(int row) { return (row & 6) | ((row >> 3) & 1); }
 
-// a column's running maximum moves only when a score exceeds it by this much (base 2): weights stay below 2^8, and the
-// accumulators are rescaled about once per column instead of at every new maximum
-constexpr float kMaxSlack = 8.f;
+// A column's weights are 2^(s - m) with m = its largest score in the first tile it sees, not a running maximum: bf16 and f32 keep
+// their relative precision at any scale, so sums and accumulators may grow with later, larger scores and are never rescaled
+// (a rescale of accumulators that fill the registers costs a copy of all of them).  Only if a score passes m by more than this
+// (base 2), the pass over the keys is repeated with m = the largest score of all.
+constexpr float kMaxGrowth = 96.f;
 
-// 32 staged rows (keys kb .. kb + 31) against CG groups of 16 columns: a row fragment read from LDS serves all groups.  m: running
-// maximum (base-2 scores; equal in the four lane groups of a column), l: this lane group's share of the sum, o: O^T
-// accumulators.  qpos < 0: column without a query.
-template <int RP, int RDP, int CG>
+// 32 staged rows (keys kb .. kb + 31) against CG groups of 16 columns: a row fragment read from LDS serves all groups.  m: the
+// column's reference (kNegBig: no key seen yet), top: its largest score so far (both base 2, equal in the four lane groups of a
+// column), l: this lane group's share of the sum, o: O^T accumulators.  qpos < 0: column without a query.
+// LDS reads as assembly with explicit waits: the fragments of a tile stream through a ring of registers several places ahead of the
+// MFMAs that use them (left to itself the compiler reads, waits and multiplies one fragment at a time when the accumulators fill
+// the registers).  LDS reads return in order, so "at most N outstanding" names the oldest ones.
+template <int OFF>
+LK_DEVICE void lds_read16(uint4_t& v, unsigned addr) {
+  asm volatile("ds_read_b128 %0, %1 offset:%2" : "=v"(v) : "v"(addr), "n"(OFF));
+}
+template <int OFF>
+LK_DEVICE void lds_read_tr(short4_t& v, unsigned addr) {
+  asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(v) : "v"(addr), "n"(OFF));
+}
+template <int N, typename V>
+LK_DEVICE void lds_wait(V& a, V& b) {
+  asm volatile("s_waitcnt lgkmcnt(%2)" : "+v"(a), "+v"(b) : "n"(N));
+}
+template <int N, int I = 0, typename F>
+LK_DEVICE void static_for(F&& f) {
+  if constexpr (I < N) {
+    f(std::integral_constant<int, I>{});
+    static_for<N, I + 1>(f);
+  }
+}
+
+// maximum over the four lane groups (lanes l, l ^ 16, l ^ 32, l ^ 48), in registers
+LK_DEVICE float max_groups(float v) {
+  // (the swapped pair is taken apart as integers: a bit cast of a vector's element reads element 0)
+  const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+  const unsigned a0 = a[0], a1 = a[1];
+  v = fmaxf(__uint_as_float(a0), __uint_as_float(a1));
+  const auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+  const unsigned b0 = b[0], b1 = b[1];
+  return fmaxf(__uint_as_float(b0), __uint_as_float(b1));
+}
+
+template <int RP, int RDP, int CG, bool THIN>
 LK_DEVICE void lat_tile(const bf16_t* tile, const uint4_t (&qf)[CG][(RP + RDP) / 32], int kb, const int (&qpos)[CG], const int (&klo)[CG], float s2,
-                        float (&m)[CG], float (&l)[CG], floatx4 (&o)[CG][RP / 16]) {
+                        float (&m)[CG], float (&top)[CG], float (&l)[CG], floatx4 (&o)[CG][RP / 16]) {
   constexpr int KD = RP + RDP, NKS = KD / 32, VT = RP / 16;
+  constexpr int QA = RP > 256 && CG == 1 && THIN ? 3 : 4, VA = 4;   // fragments requested ahead of their products (QA pairs, VA c^T fragments)
   const int lane = threadIdx.x & 63, n16 = lane & 15, g = lane >> 4;
-  const unsigned char* base = reinterpret_cast<const unsigned char*>(tile);
+  const unsigned base = (unsigned)reinterpret_cast<uintptr_t>((lds_void_ptr)tile);
   floatx4 c[CG][2];
 #pragma unroll
-  for (int t = 0; t < 2; ++t) {
+  for (int x = 0; x < CG; ++x) c[x][0] = c[x][1] = floatx4{0.f, 0.f, 0.f, 0.f};
+  const int sw = swz(n16);   // (rows n16 and 16 + n16 have the same swizzle)
+  const unsigned k0 = base + n16 * KD * 2 + (g ^ sw) * 16, k1 = base + n16 * KD * 2 + ((4 + g) ^ sw) * 16;
+  uint4_t kf[QA][2];
+  static_for<QA>([&](auto sc_) {
+    constexpr int s = decltype(sc_)::value;
+    lds_read16<128 * (s / 2)>(kf[s][0], (s & 1) ? k1 : k0);
+    lds_read16<128 * (s / 2) + 16 * KD * 2>(kf[s][1], (s & 1) ? k1 : k0);
+  });
+  static_for<NKS>([&](auto sc_) {
+    constexpr int s = decltype(sc_)::value, ahead = (s + QA < NKS ? QA : NKS - s) - 1;
+    lds_wait<2 * ahead>(kf[s % QA][0], kf[s % QA][1]);
 #pragma unroll
-    for (int x = 0; x < CG; ++x) c[x][t] = floatx4{0.f, 0.f, 0.f, 0.f};
-    const unsigned char* kr = base + (16 * t + n16) * KD * 2;
-    const int sw = swz(n16), p0 = (g ^ sw) * 16, p1 = ((4 + g) ^ sw) * 16;
+    for (int t = 0; t < 2; ++t)
 #pragma unroll
-    for (int s = 0; s < NKS; ++s) {
-      const uint4_t a = *reinterpret_cast<const uint4_t*>(kr + (s >> 1) * 128 + ((s & 1) ? p1 : p0));
-#pragma unroll
-      for (int x = 0; x < CG; ++x) c[x][t] = mma_qk<bf16_t>(a, qf[x][s], c[x][t]);
-      if (CG > 1 && s % 6 == 5) __builtin_amdgcn_sched_barrier(0);   // bounds how many fragments are in flight (registers)
+      for (int x = 0; x < CG; ++x) c[x][t] = mma_qk<bf16_t>(kf[s % QA][t], qf[x][s], c[x][t]);
+    if constexpr (s + QA < NKS) {
+      lds_read16<128 * ((s + QA) / 2)>(kf[s % QA][0], ((s + QA) & 1) ? k1 : k0);
+      lds_read16<128 * ((s + QA) / 2) + 16 * KD * 2>(kf[s % QA][1], ((s + QA) & 1) ? k1 : k0);
     }
-  }
+  });
+  // the first c^T fragments travel under the softmax arithmetic
+  const int qq = n16 >> 2, pp = n16 & 3, swv = swz(4 * g + qq);   // rows 4g + qq and 16 + 4g + qq have the same swizzle
+  const unsigned vr = base + (4 * g + qq) * KD * 2 + 8 * (pp & 1);
+  unsigned va[4];
+#pragma unroll
+  for (int x = 0; x < 4; ++x) va[x] = vr + ((2 * x + (pp >> 1)) ^ swv) * 16;
+  short4_t vlo[VA], vhi[VA];
+  static_for<VA>([&](auto vc_) {
+    constexpr int vt = decltype(vc_)::value;
+    lds_read_tr<128 * (vt / 4)>(vlo[vt], va[vt % 4]);
+    lds_read_tr<128 * (vt / 4) + 16 * KD * 2>(vhi[vt], va[vt % 4]);
+  });
   short8 pb[CG];
 #pragma unroll
   for (int x = 0; x < CG; ++x) {
@@ -95,19 +153,9 @@ LK_DEVICE void lat_tile(const bf16_t* tile, const uint4_t (&qf)[CG][(RP + RDP) /
         sc[t][j] = c[x][t][j] * s2;
         if (ok[t][j]) mx = fmaxf(mx, sc[t][j]);
       }
-    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-    if (__any(mx > m[x] + kMaxSlack)) {
-      const float mn = fmaxf(m[x], mx), alpha = __builtin_amdgcn_exp2f(m[x] - mn);
-      m[x] = mn;
-      l[x] *= alpha;
-#pragma unroll
-      for (int vt = 0; vt < VT; ++vt) {
-#pragma unroll
-        for (int j = 0; j < 4; ++j) o[x][vt][j] *= alpha;
-        if (CG > 1 && vt % 4 == 3) __builtin_amdgcn_sched_barrier(0);
-      }
-    }
+    mx = max_groups(mx);
+    if (m[x] == kNegBig) m[x] = mx;
+    top[x] = fmaxf(top[x], mx);
 #pragma unroll
     for (int t = 0; t < 2; ++t)
 #pragma unroll
@@ -117,21 +165,17 @@ LK_DEVICE void lat_tile(const bf16_t* tile, const uint4_t (&qf)[CG][(RP + RDP) /
         pb[x][4 * t + j] = (short)f2bf(p);
       }
   }
-  const int qq = n16 >> 2, pp = n16 & 3, sw = swz(4 * g + qq);   // rows 4g + qq and 16 + 4g + qq have the same swizzle
-  const unsigned char* vr = base + (4 * g + qq) * KD * 2 + 8 * (pp & 1);
-  int voff[4];
-#pragma unroll
-  for (int x = 0; x < 4; ++x) voff[x] = ((2 * x + (pp >> 1)) ^ sw) * 16;
-#pragma unroll
-  for (int vt = 0; vt < VT; ++vt) {
-    const unsigned char* a0 = vr + (vt >> 2) * 128 + voff[vt & 3];
-    const short4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4_ptr)(a0));
-    const short4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4_ptr)(a0 + 16 * KD * 2));
-    const short8 a = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
+  static_for<VT>([&](auto vc_) {
+    constexpr int vt = decltype(vc_)::value, ahead = (vt + VA < VT ? VA : VT - vt) - 1;
+    lds_wait<2 * ahead>(vlo[vt % VA], vhi[vt % VA]);
+    const short8 a = __builtin_shufflevector(vlo[vt % VA], vhi[vt % VA], 0, 1, 2, 3, 4, 5, 6, 7);
 #pragma unroll
     for (int x = 0; x < CG; ++x) o[x][vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb[x], o[x][vt], 0, 0, 0);
-    if (CG > 1 && vt % 4 == 3) __builtin_amdgcn_sched_barrier(0);
-  }
+    if constexpr (vt + VA < VT) {
+      lds_read_tr<128 * ((vt + VA) / 4)>(vlo[vt % VA], va[(vt + VA) % 4]);
+      lds_read_tr<128 * ((vt + VA) / 4) + 16 * KD * 2>(vhi[vt % VA], va[(vt + VA) % 4]);
+    }
+  });
 }
 
 template <int RP, int RDP>
@@ -141,30 +185,34 @@ LK_DEVICE void load_q(const bf16_t* qrow, bool valid, uint4_t (&qf)[(RP + RDP) /
   for (int s = 0; s < (RP + RDP) / 32; ++s) qf[s] = valid ? ld16(qrow + 32 * s + 8 * g) : uint4_t{0u, 0u, 0u, 0u};
 }
 
-// physical row of key `key` of the 16-key group kg (a multiple of 16, clamped to the sequence's last group): pages hold a
-// multiple of 16 rows, so a group lies in one page
-LK_DEVICE long group_row(const int* bt, int BS, int kg, int last) {
-  const int k = min(kg, last);
-  return (long)bt[k / BS] * BS + k % BS;
+// the page of the 16-key group kg (a multiple of 16, clamped to the sequence's last group): pages hold a multiple of 16 rows, so
+// a group lies in one page
+LK_DEVICE int group_page(const int* bt, int BS, int kg, int last) { return bt[min(kg, last) / BS]; }
+
+// 64 pieces of 16 bytes (one per lane, `src`) to 1,024 consecutive bytes of LDS at `dst` (wave-uniform), without registers.  Written as
+// assembly: the builtin makes the compiler wait for it before every transposed LDS read, also of the other buffer.  The caller
+// waits (vmcnt) before the piece is read.
+LK_DEVICE void request_piece(const void* src, void* dst) {
+  const unsigned off = __builtin_amdgcn_readfirstlane((unsigned)reinterpret_cast<uintptr_t>((lds_void_ptr)dst));
+  asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off" ::"s"(off), "v"(src) : "memory", "m0");
 }
 
 constexpr int kPreCols = 128;
 // column groups per wave: two where the accumulators of both fit the registers
 template <int RP>
-constexpr int pre_groups() { return RP <= 256 ? 2 : 1; }
+constexpr int pre_groups() { return 2; }
 template <int RP>
 constexpr int pre_waves() { return kPreCols / (16 * pre_groups<RP>()); }
 
 // grid (query tiles, head blocks): tile x is found by walking the sequences (at most ceil(qlen / NQ) tiles each, a sequence's last
 // queries first: they see the most keys)
 template <int RP, int RDP>
-__global__ __launch_bounds__(pre_waves<RP>() * 64) void lat_prefill_kernel(LatParams p, const int* __restrict__ cu_q, const int* __restrict__ ctx_lens,
+__global__ __launch_bounds__(pre_waves<RP>() * 64, RP >= 256 ? 1 : 2) void lat_prefill_kernel(LatParams p, const int* __restrict__ cu_q, const int* __restrict__ ctx_lens,
                                                                      int nseq) {
-  constexpr int KD = RP + RDP, CPR = KD / 8, VT = RP / 16, NCH = 32 * CPR, NT = pre_waves<RP>() * 64, NL = (NCH + NT - 1) / NT,
+  constexpr int KD = RP + RDP, CPR = KD / 8, VT = RP / 16, NCH = 32 * CPR, NL = (NCH / 64 + pre_waves<RP>() - 1) / pre_waves<RP>(),
                 CG = pre_groups<RP>();
-  extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
-  bf16_t* const buf = reinterpret_cast<bf16_t*>(smem);   // two tiles of 32 rows
-  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, n16 = lane & 15, g = lane >> 4;
+  extern __shared__ __attribute__((aligned(16))) unsigned char smem[];   // two tiles of 32 rows
+  const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), n16 = lane & 15, g = lane >> 4;
   const int NQ = kPreCols / p.HC;
   int b = -1, q0 = 0;
   {
@@ -184,8 +232,8 @@ __global__ __launch_bounds__(pre_waves<RP>() * 64) void lat_prefill_kernel(LatPa
   const int qbeg = cu_q[b], qlen = cu_q[b + 1] - qbeg, ctx = ctx_lens[b], past = ctx - qlen;
   uint4_t qf[CG][KD / 32];
   floatx4 o[CG][VT];
-  float m[CG], l[CG];
-  int qpos[CG], klo[CG], whi = -1, wlo = 0x7fffffff;
+  float m[CG], top[CG], l[CG];
+  int qpos[CG], klo[CG];
 #pragma unroll
   for (int x = 0; x < CG; ++x) {
     const int c = 16 * (CG * w + x) + n16, qi = q0 + c / p.HC, head = blockIdx.y * p.HC + c % p.HC;
@@ -193,50 +241,68 @@ __global__ __launch_bounds__(pre_waves<RP>() * 64) void lat_prefill_kernel(LatPa
     qpos[x] = valid ? past + qi : -1;
     klo[x] = first_key(qpos[x], p.window);
     load_q<RP, RDP>(reinterpret_cast<const bf16_t*>(p.q) + (long)(qbeg + min(qi, qlen - 1)) * p.qs + (long)min(head, p.H - 1) * KD, valid, qf[x]);
-#pragma unroll
-    for (int vt = 0; vt < VT; ++vt) o[x][vt] = floatx4{0.f, 0.f, 0.f, 0.f};
-    m[x] = p.sink && valid ? p.sink[head] * kLog2e : kNegBig;
-    l[x] = p.sink && valid && g == 0 ? 1.f : 0.f;
-    whi = max(whi, qpos[x]);
-    wlo = min(wlo, valid ? klo[x] : 0x7fffffff);
+    m[x] = kNegBig;
   }
   const float s2 = p.scale * kLog2e;
   const int k1 = min(ctx, past + q0 + NQ), k0 = first_key(past + q0, p.window) & ~31, last = (k1 - 1) & ~15;
   const int* bt = p.bt + (long)b * p.bt_stride;
   const bf16_t* cache = reinterpret_cast<const bf16_t*>(p.cache);
-  // this wave's columns see keys wlo .. whi only
-#pragma unroll
-  for (int x = 1; x < 16; x <<= 1) {
-    whi = max(whi, __shfl_xor(whi, x, 64));
-    wlo = min(wlo, __shfl_xor(wlo, x, 64));
-  }
-  uint4_t st[NL];
-  auto fetch = [&](int kb) {
-    const long r0 = group_row(bt, p.BS, kb, last), r1 = group_row(bt, p.BS, kb + 16, last);
-#pragma unroll
-    for (int i = 0; i < NL; ++i) {
-      const int x = tid + NT * i, r = x / CPR, cc = x % CPR;
-      if (NCH % NT == 0 || x < NCH) st[i] = ld16(cache + ((r < 16 ? r0 : r1) + (r & 15)) * KD + cc * 8);
-    }
-  };
-  auto stage = [&](bf16_t* dst) {
+  // a tile travels from the cache to LDS without registers (LDS-DMA): 64 pieces of 16 bytes per wave instruction, in the order of
+  // their places in LDS; the source piece of a place is the one the swizzle puts there
+  const int piece0 = 64 * w + lane;
+  constexpr int STEP = 64 * pre_waves<RP>();   // pieces per round of the workgroup's waves
+  auto request = [&](int kb, int page0, int page1, int which) {
+    const int r0 = __builtin_amdgcn_readfirstlane(page0) * p.BS + min(kb, last) % p.BS,
+              r1 = __builtin_amdgcn_readfirstlane(page1) * p.BS + min(kb + 16, last) % p.BS;
+    unsigned char* dst = smem + which * 64 * KD;
+    int r = piece0 / CPR, pos = piece0 % CPR;   // row and place of this lane's piece, stepped from instruction to instruction
+    asm volatile("" : "+v"(r), "+v"(pos));      // (recomputed per tile: the registers are worth more than the few operations)
 #pragma unroll
     for (int i = 0; i < NL; ++i) {
-      const int x = tid + NT * i, r = x / CPR, cc = x % CPR;
-      if (NCH % NT == 0 || x < NCH) *reinterpret_cast<uint4_t*>(dst + r * KD + ((cc & ~7) | ((cc & 7) ^ swz(r))) * 8) = st[i];
+      const int blk = pre_waves<RP>() * i + w;   // wave-uniform
+      if (NCH / 64 % pre_waves<RP>() == 0 || blk < NCH / 64) {
+        const int cc = (pos & ~7) | ((pos & 7) ^ swz(r));
+        request_piece(cache + (long)((r < 16 ? r0 : r1) + (r & 15)) * KD + cc * 8, dst + blk * 1024);
+      }
+      r += STEP / CPR;
+      pos += STEP % CPR;
+      if (pos >= CPR) {
+        pos -= CPR;
+        ++r;
+      }
     }
   };
-  fetch(k0);
-  stage(buf);
-  __syncthreads();
-  int cur = 0;
-  for (int kb = k0; kb < k1; kb += 32) {
-    const bool more = kb + 32 < k1;
-    if (more) fetch(kb + 32);
-    if (kb <= whi && kb + 31 >= wlo) lat_tile<RP, RDP, CG>(buf + cur * 32 * KD, qf, kb, qpos, klo, s2, m, l, o);
-    if (more) stage(buf + (cur ^ 1) * 32 * KD);
+  for (int pass = 0; pass < 2; ++pass) {
+#pragma unroll
+    for (int x = 0; x < CG; ++x) {
+      top[x] = kNegBig;
+      l[x] = 0.f;
+#pragma unroll
+      for (int vt = 0; vt < VT; ++vt) o[x][vt] = floatx4{0.f, 0.f, 0.f, 0.f};
+    }
+    request(k0, group_page(bt, p.BS, k0, last), group_page(bt, p.BS, k0 + 16, last), 0);
+    int n0 = group_page(bt, p.BS, k0 + 32, last), n1 = group_page(bt, p.BS, k0 + 48, last);   // the pages of the tile to request next
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
-    cur ^= 1;
+    int cur = 0;
+    for (int kb = k0; kb < k1; kb += 32) {
+      if (kb + 32 < k1) {
+        request(kb + 32, n0, n1, cur ^ 1);
+        n0 = group_page(bt, p.BS, kb + 64, last);   // (raw: used, and waited for, in the next round)
+        n1 = group_page(bt, p.BS, kb + 80, last);
+      }
+      lat_tile<RP, RDP, CG, true>(reinterpret_cast<const bf16_t*>(smem + cur * 64 * KD), qf, kb, qpos, klo, s2, m, top, l, o);
+      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // the next tile has arrived (this wave's part of it)
+      __syncthreads();
+      cur ^= 1;
+    }
+    int again = 0;
+#pragma unroll
+    for (int x = 0; x < CG; ++x) {
+      again |= top[x] > m[x] + kMaxGrowth;
+      m[x] = pass == 0 && top[x] > m[x] + kMaxGrowth ? top[x] : m[x];
+    }
+    if (!__syncthreads_or(again)) break;
   }
 #pragma unroll
   for (int x = 0; x < CG; ++x) {
@@ -244,6 +310,7 @@ __global__ __launch_bounds__(pre_waves<RP>() * 64) void lat_prefill_kernel(LatPa
     l[x] += __shfl_xor(l[x], 32, 64);
     const int c = 16 * (CG * w + x) + n16, qi = q0 + c / p.HC, head = blockIdx.y * p.HC + c % p.HC;
     if (qpos[x] >= 0) {
+      if (p.sink) l[x] += __builtin_amdgcn_exp2f(p.sink[head] * kLog2e - m[x]);   // one more term without a value
       const float f = l[x] > 0.f ? 1.f / l[x] : 0.f;
       bf16_t* orow = reinterpret_cast<bf16_t*>(p.out) + (long)(qbeg + qi) * p.os + (long)head * RP + 4 * g;
 #pragma unroll
@@ -272,27 +339,32 @@ __global__ __launch_bounds__(256) void lat_decode_kernel(LatParams p, const int*
   uint4_t qf[1][KD / 32];
   load_q<RP, RDP>(qrow, valid, qf[0]);
   floatx4 o[1][VT];
-#pragma unroll
-  for (int vt = 0; vt < VT; ++vt) o[0][vt] = floatx4{0.f, 0.f, 0.f, 0.f};
-  const bool own_sink = p.sink && valid && z == 0 && w == 0;
-  float m[1] = {own_sink ? p.sink[head] * kLog2e : kNegBig}, l[1] = {own_sink && g == 0 ? 1.f : 0.f};
+  float m[1] = {kNegBig}, top[1], l[1];
   const float s2 = p.scale * kLog2e;
   const int nsteps = ctx > 0 ? (ctx - k0 + 31) / 32 : 0, spz = (nsteps + Z - 1) / Z, e1 = min(nsteps, (z + 1) * spz);
   const int* bt = p.bt + (long)b * p.bt_stride;
   const bf16_t* cache = reinterpret_cast<const bf16_t*>(p.cache);
-  for (int step = z * spz + w; step < e1; step += 4) {
-    const int kb = k0 + 32 * step;
-    // tiles start at the first visible key (a window of 32 n keys is n tiles): lane x looks up the cache row of key kb + x % 32
-    const int key = min(kb + (lane & 31), ctx - 1), mine = bt[key / p.BS] * p.BS + key % p.BS;
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // the previous tile's LDS reads are done
+  for (int pass = 0; pass < 2; ++pass) {
+    top[0] = kNegBig;
+    l[0] = 0.f;
 #pragma unroll
-    for (int i = 0; i < NCH / 64; ++i) {
-      // LDS piece x = 64 i + lane of the region is position x % CPR of row x / CPR: it holds the source piece swizzled back
-      const int x = 64 * i + lane, r = x / CPR, pos = x % CPR, cc = (pos & ~7) | ((pos & 7) ^ swz(r));
-      __builtin_amdgcn_global_load_lds((gbl_void_ptr)(cache + (long)__shfl(mine, r, 64) * KD + cc * 8), (lds_void_ptr)(region + i * 1024), 16, 0, 0);
+    for (int vt = 0; vt < VT; ++vt) o[0][vt] = floatx4{0.f, 0.f, 0.f, 0.f};
+    for (int step = z * spz + w; step < e1; step += 4) {
+      const int kb = k0 + 32 * step;
+      // tiles start at the first visible key (a window of 32 n keys is n tiles): lane x looks up the cache row of key kb + x % 32
+      const int key = min(kb + (lane & 31), ctx - 1), mine = bt[key / p.BS] * p.BS + key % p.BS;
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // the previous tile's LDS reads are done
+  #pragma unroll
+      for (int i = 0; i < NCH / 64; ++i) {
+        // LDS piece x = 64 i + lane of the region is position x % CPR of row x / CPR: it holds the source piece swizzled back
+        const int x = 64 * i + lane, r = x / CPR, pos = x % CPR, cc = (pos & ~7) | ((pos & 7) ^ swz(r));
+        __builtin_amdgcn_global_load_lds((gbl_void_ptr)(cache + (long)__shfl(mine, r, 64) * KD + cc * 8), (lds_void_ptr)(region + i * 1024), 16, 0, 0);
+      }
+      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+      lat_tile<RP, RDP, 1, false>(reinterpret_cast<const bf16_t*>(region), qf, kb, qpos, klo, s2, m, top, l, o);
     }
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    lat_tile<RP, RDP, 1>(reinterpret_cast<const bf16_t*>(region), qf, kb, qpos, klo, s2, m, l, o);
+    if (!__any(top[0] > m[0] + kMaxGrowth)) break;
+    m[0] = top[0] > m[0] + kMaxGrowth ? top[0] : m[0];
   }
   // ---- merge the 4 waves: (m, l) behind every region's O block, then O relative to the common maximum
   l[0] += __shfl_xor(l[0], 16, 64);
@@ -304,7 +376,9 @@ __global__ __launch_bounds__(256) void lat_decode_kernel(LatParams p, const int*
     ml[16 + n16] = l[0];
   }
   __syncthreads();
-  float M = kNegBig, L = 0.f;
+  // (the sink is one more term without a value, counted by the first split)
+  const float sk = p.sink && z == 0 ? p.sink[min(head, p.H - 1)] * kLog2e : kNegBig;
+  float M = sk, L = 0.f;
 #pragma unroll
   for (int i = 0; i < 4; ++i) M = fmaxf(M, reinterpret_cast<const float*>(smem + i * 64 * KD + 64 * RP)[n16]);
 #pragma unroll
@@ -312,6 +386,7 @@ __global__ __launch_bounds__(256) void lat_decode_kernel(LatParams p, const int*
     const float* q = reinterpret_cast<const float*>(smem + i * 64 * KD + 64 * RP);
     L += q[16 + n16] * __builtin_amdgcn_exp2f(q[n16] - M);
   }
+  if (p.sink && z == 0) L += __builtin_amdgcn_exp2f(sk - M);
   const float f = __builtin_amdgcn_exp2f(m[0] - M);
   floatx4* ob = reinterpret_cast<floatx4*>(region);
 #pragma unroll

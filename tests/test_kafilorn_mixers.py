@@ -256,6 +256,48 @@ def test_latent_attention_of_many_shapes(H, R, rd, window, bs, device, dtype):
             assert rel_err(out, want) < tol(dtype), (Z, rel_err(out, want))
 
 
+@pytest.mark.parametrize("device,dtype", ALL)
+@pytest.mark.parametrize("H,R,window", [(4, 96, 0), (16, 128, 45), (5, 200, 61), (16, 500, 0), (3, 512, 70), (2, 600, 50)])
+def test_latent_attention_with_scores_that_climb_and_fall_far(H, R, window, device, dtype):
+    """Scores that pass those of the first keys by 50 and then by 90 or 160 nats (head by head also falling, and level): the
+    weights stay those of a softmax over all keys, whichever tile the largest score lies in, for prompts cut anywhere
+    and for decoded rows with 1 to 3 key splits."""
+    g = torch.Generator().manual_seed(R)
+    rp, rdp = ops.latent_row(R, 16)
+    KD, n, scale = rp + rdp, 130, 0.25
+    level = torch.zeros(n, dtype=torch.float64)
+    level[40:77], level[77:], level[101], level[118:] = 50.0, 90.0, 160.0, 158.0
+    rows = torch.zeros(n, KD, dtype=torch.float64)
+    rows[:, :R], rows[:, rp] = q16(rnd(g, n, R)), q16(level / scale)
+    bt = torch.randperm(12, generator=g)[:9].to(torch.int32)[None]
+    cache = torch.zeros(12, BS, KD, dtype=torch.float64)
+    for i in range(n):
+        cache[int(bt[0, i // BS]), i % BS] = rows[i]
+    qa = torch.zeros(n, H, KD, dtype=torch.float64)
+    qa[..., :R] = q16(rnd(g, n, H, R, scale=1.0 / math.sqrt(R)))
+    qa[..., rp] = torch.tensor([1.0, -1.0, 0.0])[torch.arange(H) % 3]
+    sink = (2.0 * torch.arange(H) - 3.0).float()
+    sink[0] = 60.0
+    s = torch.einsum("qhk,jk->qhj", qa, rows) * scale
+    d = torch.arange(n)[:, None] - torch.arange(n)[None]
+    s = s.masked_fill(((d < 0) | ((d >= window) if window else (d < 0)))[:, None], -math.inf)
+    full = torch.cat([s, sink.double()[None, :, None].expand(n, H, 1)], -1)
+    want = torch.einsum("qhj,jr->qhr", torch.softmax(full, -1)[..., :-1], rows[:, :rp])
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=device)   # noqa: E731
+    dev = lambda t: t.to(dtype).to(device)   # noqa: E731
+    for lo, hi in ((0, n), (0, 41), (41, 78), (78, 103), (103, n)):
+        out = torch.empty(hi - lo, H, rp, dtype=dtype, device=device)
+        ops.latent_attention_prefill(dev(qa[lo:hi]), dev(cache), bt.to(device), i32([0, hi - lo]), i32([hi]), window, scale, sink.to(device), rp, out,
+                                     hi - lo)
+        assert rel_err(out, want[lo:hi]) < tol(dtype), (lo, hi, rel_err(out, want[lo:hi]))
+    at = [1, 41, 78, 102, 103, 119, n]
+    for Z in (1, 2, 3):
+        out = torch.empty(len(at), H, rp, dtype=dtype, device=device)
+        ops.latent_attention_decode(dev(qa[[a - 1 for a in at]]), dev(cache), bt.expand(len(at), -1).contiguous().to(device), i32(at), window, scale,
+                                    sink.to(device), rp, out, splits=Z)
+        assert rel_err(out, want[[a - 1 for a in at]]) < tol(dtype), (Z, rel_err(out, want[[a - 1 for a in at]]))
+
+
 def scan_reference(q, k, v, ig, f, scale):
     """q, k [T, H, dk], v [T, H, dv], gates [T, H] (log domain), one sequence from zero."""
     T, H, dk = q.shape
