@@ -81,6 +81,11 @@ LK_DEVICE void store8(bf16_t* p, const float* f) {
 }
 
 // Activations shared by the elementwise kernels and the GEMM epilogues.
+// the pair (a, b) turned by an angle: (a c - b s, b c + a s), one product rounded before the fma.  Written out, so that every kernel
+// that rotates (alone or in a product's epilogue) rounds alike.
+LK_DEVICE float rot_lo(float a, float b, float c, float s) { return __builtin_fmaf(a, c, -(b * s)); }
+LK_DEVICE float rot_hi(float a, float b, float c, float s) { return __builtin_fmaf(b, c, a * s); }
+
 LK_DEVICE float lk_silu(float x) { return x / (1.f + __expf(-x)); }
 // erf by Abramowitz & Stegun 7.1.26 (|error| <= 1.5e-7, far below bf16's 2^-9): one
 // hardware exp + one reciprocal + a 5-term Horner polynomial.  The library erff made the

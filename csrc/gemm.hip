@@ -634,8 +634,8 @@ __device__ __forceinline__ void gemm8_body(const bf16_t* __restrict__ X, long ld
           }
           for (int q = 0; q < n / 2; ++q) {
             const float a = y[2 * q], b = y[2 * q + 1];
-            y[2 * q] = a * cv[q] - b * sv[q];
-            y[2 * q + 1] = b * cv[q] + a * sv[q];
+            y[2 * q] = rot_lo(a, b, cv[q], sv[q]);
+            y[2 * q + 1] = rot_hi(a, b, cv[q], sv[q]);
           }
         }
         uint4_t pk;

@@ -492,8 +492,8 @@ __global__ __launch_bounds__(256, 1) void gemm1w_kernel(const bf16_t* __restrict
 #pragma unroll
               for (int q = 0; q < 4; ++q) {
                 const float a = y[2 * q], b = y[2 * q + 1];
-                y[2 * q] = a * c4[p][q] - b * s4[p][q];
-                y[2 * q + 1] = b * c4[p][q] + a * s4[p][q];
+                y[2 * q] = rot_lo(a, b, c4[p][q], s4[p][q]);
+                y[2 * q + 1] = rot_hi(a, b, c4[p][q], s4[p][q]);
               }
             }
             const u32x4_t pk = pk8(y);

@@ -293,7 +293,7 @@ __global__ __launch_bounds__(256) void gemv_decode_kernel(GemvArgs g) {
         } else {
           const float* cs = g.cos_sin + (long)g.positions[m] * g.D;  // [cos(D/2) | sin(D/2)]
           const float c = cs[ip], s = cs[hd + ip];
-          const float y1 = x1 * c - x2 * s, y2 = x2 * c + x1 * s;
+          const float y1 = rot_lo(x1, x2, c, s), y2 = rot_hi(x1, x2, c, s);
           if (head < g.Hq) {
             orow[ra] = f2bf(y1);
             orow[rb] = f2bf(y2);

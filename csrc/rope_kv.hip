@@ -102,8 +102,8 @@ __global__ __launch_bounds__(64) void rope_kv_kernel(
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
       const float c = j < 4 ? c0[j] : c1[j - 4], s = j < 4 ? s0[j] : s1[j - 4];
-      y1[j] = x1[j] * c - x2[j] * s;
-      y2[j] = x2[j] * c + x1[j] * s;
+      y1[j] = rot_lo(x1[j], x2[j], c, s);
+      y2[j] = rot_hi(x1[j], x2[j], c, s);
     }
     if (store_src) {
       store8(hp + i0, y1);
@@ -122,8 +122,8 @@ __global__ __launch_bounds__(64) void rope_kv_kernel(
     const floatx4 s4 = *reinterpret_cast<const floatx4*>(cs + half + (e0 >> 1));
 #pragma unroll
     for (int p = 0; p < 4; ++p) {
-      y[2 * p] = x[2 * p] * c4[p] - x[2 * p + 1] * s4[p];
-      y[2 * p + 1] = x[2 * p + 1] * c4[p] + x[2 * p] * s4[p];
+      y[2 * p] = rot_lo(x[2 * p], x[2 * p + 1], c4[p], s4[p]);
+      y[2 * p + 1] = rot_hi(x[2 * p], x[2 * p + 1], c4[p], s4[p]);
     }
     if (store_src) store8(hp + e0, y);
     if (kdst) store8(kdst + e0, y);

@@ -228,8 +228,8 @@ LK_DEVICE void tail_rope_kv(const WsTail& tl, __amdgpu_buffer_rsrc_t prs, int S,
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
         const float c = cs[i0 + j], sn = cs[half + i0 + j];
-        y1[j] = x1[j] * c - x2[j] * sn;
-        y2[j] = x2[j] * c + x1[j] * sn;
+        y1[j] = rot_lo(x1[j], x2[j], c, sn);
+        y2[j] = rot_hi(x1[j], x2[j], c, sn);
       }
       store8(hp + i0, store_src ? y1 : x1);
       store8(hp + half + i0, store_src ? y2 : x2);
@@ -244,8 +244,8 @@ LK_DEVICE void tail_rope_kv(const WsTail& tl, __amdgpu_buffer_rsrc_t prs, int S,
 #pragma unroll
       for (int p = 0; p < 4; ++p) {
         const float c = cs[(e0 >> 1) + p], sn = cs[half + (e0 >> 1) + p];
-        y[2 * p] = x[2 * p] * c - x[2 * p + 1] * sn;
-        y[2 * p + 1] = x[2 * p + 1] * c + x[2 * p] * sn;
+        y[2 * p] = rot_lo(x[2 * p], x[2 * p + 1], c, sn);
+        y[2 * p + 1] = rot_hi(x[2 * p], x[2 * p + 1], c, sn);
       }
       store8(hp + e0, store_src ? y : x);
       if (kdst) store8(kdst + e0, y);
