@@ -74,6 +74,10 @@ CONFIGS = {
     "wide": config([dense(lat(18, 12, 10, 8, 40, 140, 0.2, 10000.0, 4096), 24),
                     moe(mls(1, 72, 100, 15.0), 24, 4, 2, 4, 2, 8),
                     dense(lat(17, 16, 10, 12, 24, 140, 0.2, 10000.0, 16, kv_from=0), 50)], 56, 8, vocab=130, escale=3.0, lscale=0.25),
+    # attention layers alone (no recurrent state, pages only), without feed-forwards and with one group kept of one
+    "pages": config([bare(lat(2, 6, 8, 8, 10, 16, 0.4, 50.0, 12)), moe(lat(3, 9, 8, 7, 11, 16, 0.3, 50.0, 25, kv_from=0), 12, 5, 2, 1, 1, 10)], 44, 2),
+    # matrix memories alone (state slots only, nothing is cached per token)
+    "slots": config([bare(mls(2, 9, 13, 4.0)), dense(mls(3, 16, 6, 20.0), 18)], 40, 5, vocab=70),
     # projections the MFMA / weight-streaming kernels tile: no vendor GEMM, decode steps captured in hipGraphs
     "mid": config([dense(mls(4, 64, 64, 12.0), 256),
                    moe(lat(4, 64, 32, 64, 256, 224, 0.1, 10000.0, 48), 128, 8, 2, 4, 2, 256),
@@ -150,7 +154,7 @@ def test_whole_prompt_streams_and_logits(name, device, dtype):
 
 
 @pytest.mark.parametrize("device,dtype", ALL)
-@pytest.mark.parametrize("name", ["tri", "odd", "wide"])
+@pytest.mark.parametrize("name", ["tri", "odd", "wide", "pages", "slots"])
 def test_prefill_equals_token_by_token_and_portions(name, device, dtype):
     """One step for the whole prompt, one token per step, and portions of changing size down to two tokens
     (cut inside pages and windows) give the same logits at every position."""
@@ -252,7 +256,7 @@ def test_long_decode_through_pages_and_windows(device, dtype):
 
 
 @pytest.mark.parametrize("device,dtype", ALL)
-@pytest.mark.parametrize("name", ["tri", "wide"])
+@pytest.mark.parametrize("name", ["tri", "wide", "pages", "slots"])
 def test_greedy_generation_through_the_scheduler(name, device, dtype):
     """``LLMEngine.generate``: the scheduler admits, chunks (a 24-token step budget) and batches three
     prompts; every generated token must be the oracle's argmax for its prefix (or within a near tie)."""
