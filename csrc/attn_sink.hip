@@ -60,6 +60,7 @@ struct SinkParams {
   int pool;
   int keep;             // window masks: positions below `keep` stay visible behind the window
   float cap;            // > 0: scores become cap * tanh(score / cap)
+  float oscale;         // multiplies every output
   int gelem;            // the gate has one column per output element (gcol + h * vdim + d) instead of one per head
 };
 
@@ -316,7 +317,7 @@ __global__ __launch_bounds__(256) void sinkattn_prefill_kernel(SinkParams p, con
   }
   if ((WT || w == 0) && cvalid) {
     const float den = l + (p.sink ? exp_f<EXACT>(-m) : 0.f);
-    const float f = den > 0.f ? gate_of<T>(p, qbeg + qi, head) / den : 0.f;
+    const float f = den > 0.f ? p.oscale * gate_of<T>(p, qbeg + qi, head) / den : 0.f;
     T* orow = out + (long)(qbeg + qi) * os + (long)head * p.vdim;
 #pragma unroll
     for (int vt = 0; vt < VT; ++vt)
@@ -368,7 +369,7 @@ __global__ __launch_bounds__(256) void sinkattn_decode_kernel(SinkParams p, cons
   if (w == 0 && cvalid) {
     if (Z == 1) {
       const float den = l + (p.sink ? exp_f<EXACT>(-m) : 0.f);
-      const float f = den > 0.f ? gate_of<T>(p, b, head) / den : 0.f;
+      const float f = den > 0.f ? p.oscale * gate_of<T>(p, b, head) / den : 0.f;
 #pragma unroll
       for (int vt = 0; vt < VT; ++vt)
 #pragma unroll
@@ -403,7 +404,7 @@ __global__ __launch_bounds__(256) void sinkattn_reduce_kernel(SinkParams p, cons
   for (int z = 0; z < Z; ++z) M = fmaxf(M, pp[(long)z * (p.vdim + 2) + p.vdim]);
   float den = p.sink ? exp_f<EXACT>(-M) : 0.f;
   for (int z = 0; z < Z; ++z) den += pp[(long)z * (p.vdim + 2) + p.vdim + 1] * exp_f<EXACT>(pp[(long)z * (p.vdim + 2) + p.vdim] - M);
-  const float f = den > 0.f ? gate_of<T>(p, b, head) / den : 0.f;
+  const float f = den > 0.f ? p.oscale * gate_of<T>(p, b, head) / den : 0.f;
   for (int vd = threadIdx.x; vd < p.vdim; vd += 256) {
     float s = 0.f;
     for (int z = 0; z < Z; ++z) s += pp[(long)z * (p.vdim + 2) + vd] * exp_f<EXACT>(pp[(long)z * (p.vdim + 2) + p.vdim] - M);
@@ -554,11 +555,11 @@ int decode_t(const SinkParams& p, const int* ctx, int B, int Z, void* out, long 
 
 SinkParams make_params(const void* q, long qs, const void* kc, const void* vc, const int* bt, int bt_stride, int H, int G, int dim,
                        int vdim, int BS, const float* hscale, int mkind, int msize, int sink, const void* gate, long gs, int gcol,
-                       const void* pkc, const void* pvc, int pool, int keep, float cap, int gelem) {
+                       const void* pkc, const void* pvc, int pool, int keep, float cap, int gelem, float oscale) {
   SinkParams p;
   p.q = q; p.qs = qs; p.kc = kc; p.vc = vc; p.bt = bt; p.bt_stride = bt_stride;
   p.H = H; p.G = G; p.dim = dim; p.vdim = vdim; p.BS = BS; p.hscale = hscale; p.mkind = mkind; p.msize = msize; p.sink = sink;
-  p.gate = gate; p.gs = gs; p.gcol = gcol; p.pkc = pkc; p.pvc = pvc; p.pool = pool; p.keep = keep; p.cap = cap; p.gelem = gelem;
+  p.gate = gate; p.gs = gs; p.gcol = gcol; p.pkc = pkc; p.pvc = pvc; p.pool = pool; p.keep = keep; p.cap = cap; p.gelem = gelem; p.oscale = oscale;
   return p;
 }
 
@@ -584,10 +585,10 @@ int lk_normrope_kv_write(void* qkv, long qs, long T, int H, int G, int dim, int 
 int lk_sinkattn_prefill(const void* q, long qs, const void* kc, const void* vc, const int* bt, int bt_stride, const int* cu_q,
                         const int* ctx_lens, const int* tile_seq, const int* tile_q0, int ntiles, int H, int G, int dim, int vdim,
                         int BS, const float* hscale, int mkind, int msize, int sink, const void* gate, long gs, int gcol, void* out,
-                        long os, const void* pkc, const void* pvc, int pool, int keep, float cap, int gelem, int esz, hipStream_t st) {
+                        long os, const void* pkc, const void* pvc, int pool, int keep, float cap, int gelem, float oscale, int esz, hipStream_t st) {
   if (ntiles <= 0) return 0;
   const SinkParams p = make_params(q, qs, kc, vc, bt, bt_stride, H, G, dim, vdim, BS, hscale, mkind, msize, sink, gate, gs, gcol, pkc, pvc,
-                                   pool, keep, cap, gelem);
+                                   pool, keep, cap, gelem, oscale);
   if (!shape_ok(p, esz)) return -1;
   return esz == 2 ? prefill_t<bf16_t>(p, cu_q, ctx_lens, tile_seq, tile_q0, ntiles, out, os, st)
                   : prefill_t<float>(p, cu_q, ctx_lens, tile_seq, tile_q0, ntiles, out, os, st);
@@ -596,10 +597,10 @@ int lk_sinkattn_prefill(const void* q, long qs, const void* kc, const void* vc, 
 int lk_sinkattn_decode(const void* q, long qs, const void* kc, const void* vc, const int* bt, int bt_stride, const int* ctx_lens,
                        int B, int Z, int H, int G, int dim, int vdim, int BS, const float* hscale, int mkind, int msize, int sink,
                        const void* gate, long gs, int gcol, void* out, long os, float* part, const void* pkc, const void* pvc,
-                       int pool, int keep, float cap, int gelem, int esz, hipStream_t st) {
+                       int pool, int keep, float cap, int gelem, float oscale, int esz, hipStream_t st) {
   if (B <= 0) return 0;
   const SinkParams p = make_params(q, qs, kc, vc, bt, bt_stride, H, G, dim, vdim, BS, hscale, mkind, msize, sink, gate, gs, gcol, pkc, pvc,
-                                   pool, keep, cap, gelem);
+                                   pool, keep, cap, gelem, oscale);
   if (!shape_ok(p, esz) || Z < 1 || (Z > 1 && part == nullptr)) return -1;
   return esz == 2 ? decode_t<bf16_t>(p, ctx_lens, B, Z, out, os, part, st) : decode_t<float>(p, ctx_lens, B, Z, out, os, part, st);
 }

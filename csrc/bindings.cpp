@@ -1470,7 +1470,7 @@ void sinkattn_prefill(const at::Tensor& q, const at::Tensor& kc, const at::Tenso
                       int64_t vdim, const at::Tensor& hscale, int64_t mkind, int64_t msize, bool sink,
                       const c10::optional<at::Tensor>& gate, int64_t gate_col, at::Tensor& out,
                       const c10::optional<at::Tensor>& pkc, const c10::optional<at::Tensor>& pvc, int64_t pool, int64_t keep_first,
-                      double softcap, bool gate_elem) {
+                      double softcap, bool gate_elem, double out_scale) {
   CHECK_CUDA(q); CHECK_LASTDIM(q); CHECK_CUDA(out); CHECK_LASTDIM(out);
   const int esz = esz_of(q, "q");
   const void *pkp = nullptr, *pvp = nullptr;
@@ -1489,7 +1489,7 @@ void sinkattn_prefill(const at::Tensor& q, const at::Tensor& kc, const at::Tenso
   CHECK_RC(lk_sinkattn_prefill(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), ip(bt), (int)bt.stride(0), ip(cu_q), ip(ctx),
                                ip(tile_seq), ip(tile_q0), (int)tile_seq.numel(), (int)H, (int)G, (int)dim, (int)vdim, (int)kc.size(2),
                                fp(hscale, H, "hscale"), (int)mkind, (int)msize, sink ? 1 : 0, gp, gs, (int)gate_col, out.data_ptr(),
-                               out.stride(0), pkp, pvp, (int)pool, (int)keep_first, (float)softcap, gate_elem ? 1 : 0, esz, cur_stream()),
+                               out.stride(0), pkp, pvp, (int)pool, (int)keep_first, (float)softcap, gate_elem ? 1 : 0, (float)out_scale, esz, cur_stream()),
            "sinkattn_prefill");
 }
 
@@ -1497,7 +1497,7 @@ void sinkattn_decode(const at::Tensor& q, const at::Tensor& kc, const at::Tensor
                      int64_t Z, int64_t H, int64_t G, int64_t dim, int64_t vdim, const at::Tensor& hscale, int64_t mkind,
                      int64_t msize, bool sink, const c10::optional<at::Tensor>& gate, int64_t gate_col, at::Tensor& out,
                      const c10::optional<at::Tensor>& part, const c10::optional<at::Tensor>& pkc,
-                     const c10::optional<at::Tensor>& pvc, int64_t pool, int64_t keep_first, double softcap, bool gate_elem) {
+                     const c10::optional<at::Tensor>& pvc, int64_t pool, int64_t keep_first, double softcap, bool gate_elem, double out_scale) {
   CHECK_CUDA(q); CHECK_LASTDIM(q); CHECK_CUDA(out); CHECK_LASTDIM(out);
   const int esz = esz_of(q, "q");
   const void *pkp = nullptr, *pvp = nullptr;
@@ -1521,7 +1521,7 @@ void sinkattn_decode(const at::Tensor& q, const at::Tensor& kc, const at::Tensor
   CHECK_RC(lk_sinkattn_decode(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), ip(bt), (int)bt.stride(0), ip(ctx), (int)B, (int)Z,
                               (int)H, (int)G, (int)dim, (int)vdim, (int)kc.size(2), fp(hscale, H, "hscale"), (int)mkind, (int)msize,
                               sink ? 1 : 0, gp, gs, (int)gate_col, out.data_ptr(), out.stride(0), pp, pkp, pvp, (int)pool, (int)keep_first,
-                              (float)softcap, gate_elem ? 1 : 0, esz, cur_stream()),
+                              (float)softcap, gate_elem ? 1 : 0, (float)out_scale, esz, cur_stream()),
            "sinkattn_decode");
 }
 
@@ -1831,6 +1831,154 @@ std::vector<at::Tensor> router_choice(const at::Tensor& h, const at::Tensor& w, 
   return {experts, weights};
 }
 
+// ---------------------------------------------------------------------------------------------
+// causal attention with biased projections and element gates, gated delta rule with one decay per head, sandwiched layer norms
+at::Tensor stream_sandwich_layernorm(at::Tensor& x, const c10::optional<at::Tensor>& y, const c10::optional<at::Tensor>& w_post,
+                                     const c10::optional<at::Tensor>& b_post, const c10::optional<at::Tensor>& add, const at::Tensor& w,
+                                     const at::Tensor& b, double eps, const c10::optional<at::Tensor>& idx, at::ScalarType out_dtype) {
+  CHECK_CUDA(x); CHECK_F32(x); CHECK_CONTIG(x);
+  TORCH_CHECK(x.dim() == 2, "x must be [T, W]");
+  TORCH_CHECK(out_dtype == at::kBFloat16 || out_dtype == at::kFloat, "out dtype");
+  const long T = x.size(0);
+  const int W = x.size(1);
+  long ys = 0;
+  int yesz = 4;
+  if (y) {
+    CHECK_CUDA(*y); CHECK_LASTDIM(*y);
+    yesz = esz_of(*y, "y");
+    TORCH_CHECK(y->dim() == 2 && y->size(0) == T && y->size(1) == W, "y shape");
+    TORCH_CHECK(w_post.has_value() && b_post.has_value(), "the sublayer norm's weight and bias");
+    ys = y->stride(0);
+  }
+  if (idx) { CHECK_CUDA(*idx); TORCH_CHECK(idx->scalar_type() == at::kLong && idx->is_contiguous(), "idx must be int64"); }
+  at::Tensor out = at::empty({idx ? idx->numel() : T, W}, x.options().dtype(out_dtype));
+  CHECK_RC(lk_stream_sandwich(x.data_ptr<float>(), y ? y->data_ptr() : nullptr, ys, yesz, fpo(w_post, W, "w_post"), fpo(b_post, W, "b_post"),
+                              fpo(add, W, "add"), fp(w, W, "w"), fp(b, W, "b"), (float)eps, idx ? idx->data_ptr<int64_t>() : nullptr,
+                              out.size(0), out.data_ptr(), out.stride(0), (int)out.element_size(), W, cur_stream()),
+           "stream_sandwich_layernorm");
+  return out;
+}
+
+void qkv_file(at::Tensor& u, int64_t col0, int64_t H, int64_t G, int64_t dim, int64_t vdim, const c10::optional<at::Tensor>& bias,
+              const c10::optional<at::Tensor>& qw, const c10::optional<at::Tensor>& kw, int64_t norm_q, int64_t norm_k, double eps, int64_t rot,
+              const c10::optional<at::Tensor>& freq, double mag, const at::Tensor& positions, at::Tensor& kc, at::Tensor& vc,
+              const at::Tensor& slots) {
+  CHECK_CUDA(u); CHECK_LASTDIM(u); CHECK_CUDA(slots); CHECK_I32(slots); CHECK_CONTIG(slots); CHECK_CUDA(positions); CHECK_I32(positions);
+  CHECK_CONTIG(positions);
+  const int esz = esz_of(u, "u");
+  const long T = u.size(0);
+  TORCH_CHECK(H >= 1 && G >= 1 && dim >= 1 && vdim >= 1, "sizes");
+  const int64_t n = (H + G) * dim + G * vdim;
+  TORCH_CHECK(u.dim() == 2 && col0 >= 0 && u.size(1) >= col0 + n, "u must hold q | k | v");
+  TORCH_CHECK(slots.numel() >= T && positions.numel() >= T, "slots / positions");
+  TORCH_CHECK(rot >= 0 && rot % 2 == 0 && rot <= dim && (rot == 0 || freq.has_value()), "rot");
+  check_sig_caches(u, kc, vc, G, dim, vdim);
+  CHECK_RC(lk_qkv_file((char*)u.data_ptr() + col0 * esz, u.stride(0), T, (int)H, (int)G, (int)dim, (int)vdim, fpo(bias, n, "bias"),
+                       fpo(qw, H * dim, "q norm weight"), fpo(kw, G * dim, "k norm weight"), (int)norm_q, (int)norm_k, (float)eps, (int)rot,
+                       rot ? fpo(freq, rot / 2, "freq") : nullptr, (float)mag, ip(positions), kc.data_ptr(), vc.data_ptr(), ip(slots),
+                       (int)kc.size(2), esz, cur_stream()), "qkv_file");
+}
+
+// what the three kernels have in common: query rows, caches of G heads, tables, gate
+void check_diff_inputs(const at::Tensor& q, const at::Tensor& kc, const at::Tensor& vc, const at::Tensor& bt, const at::Tensor& ctx, int64_t maps,
+                       int64_t H, int64_t G, int64_t dim, int64_t vdim, const at::Tensor& out) {
+  CHECK_CUDA(q); CHECK_LASTDIM(q); CHECK_CUDA(out); CHECK_LASTDIM(out);
+  esz_of(q, "q");
+  same_type(out, q, "out");
+  TORCH_CHECK(H >= 1 && G >= 1 && H % G == 0 && dim >= 1 && vdim >= 1, "sizes");
+  TORCH_CHECK(q.dim() == 2 && q.size(1) >= H * maps * dim && out.dim() == 2 && out.size(0) == q.size(0) && out.size(1) >= H * vdim, "q / out shape");
+  check_rows16(q, "q");
+  check_sig_caches(q, kc, vc, G, maps * dim, vdim);
+  CHECK_CUDA(bt); CHECK_I32(bt); CHECK_CUDA(ctx); CHECK_I32(ctx); CHECK_CONTIG(ctx);
+  TORCH_CHECK(bt.dim() == 2 && bt.stride(1) == 1, "block tables");
+}
+
+void check_tiles(const at::Tensor& bt, const at::Tensor& cu_q, const at::Tensor& ctx, const at::Tensor& ts, const at::Tensor& tq) {
+  CHECK_CUDA(cu_q); CHECK_I32(cu_q); CHECK_CONTIG(cu_q); CHECK_CUDA(ts); CHECK_I32(ts); CHECK_CONTIG(ts); CHECK_CUDA(tq); CHECK_I32(tq); CHECK_CONTIG(tq);
+  TORCH_CHECK(bt.size(0) >= cu_q.numel() - 1 && ctx.numel() >= cu_q.numel() - 1 && tq.numel() == ts.numel(), "block tables / lengths / tiles");
+}
+
+void diff_attention_prefill(const at::Tensor& q, const at::Tensor& kc, const at::Tensor& vc, const at::Tensor& bt, const at::Tensor& cu_q,
+                            const at::Tensor& ctx, const at::Tensor& ts, const at::Tensor& tq, int64_t H, int64_t G, int64_t dim, int64_t vdim,
+                            double scale, double tcoef, int64_t tevery, const at::Tensor& lam, double eps, int64_t norm_vdim, double oscale,
+                            const at::Tensor& gate, int64_t gate_col, at::Tensor& out) {
+  check_diff_inputs(q, kc, vc, bt, ctx, 2, H, G, dim, vdim, out);
+  check_tiles(bt, cu_q, ctx, ts, tq);
+  long gs = 0;
+  const void* gp = gate_rows(gate, q, gate_col, H * vdim, &gs);
+  CHECK_RC(lk_diff_attention_prefill(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), ip(bt), (int)bt.stride(0), ip(cu_q), ip(ctx), ip(ts),
+                                     ip(tq), (int)ts.numel(), (int)H, (int)G, (int)dim, (int)vdim, (int)kc.size(2), (float)scale, (float)tcoef,
+                                     (int)tevery, fp(lam, 1, "lam"), (float)eps, (int)norm_vdim, (float)oscale, gp, gs, (int)gate_col,
+                                     out.data_ptr(), out.stride(0), esz_of(q, "q"), cur_stream()), "diff_attention_prefill");
+}
+
+void diff_attention_decode(const at::Tensor& q, const at::Tensor& kc, const at::Tensor& vc, const at::Tensor& bt, const at::Tensor& ctx, int64_t Z,
+                           int64_t H, int64_t G, int64_t dim, int64_t vdim, double scale, double tcoef, int64_t tevery, const at::Tensor& lam,
+                           double eps, int64_t norm_vdim, double oscale, const at::Tensor& gate, int64_t gate_col, at::Tensor& out,
+                           const c10::optional<at::Tensor>& part) {
+  check_diff_inputs(q, kc, vc, bt, ctx, 2, H, G, dim, vdim, out);
+  const long B = q.size(0);
+  TORCH_CHECK(bt.size(0) >= B && ctx.numel() >= B && Z >= 1 && Z <= 65535, "block tables / lengths / splits");
+  float* pp = nullptr;
+  if (Z > 1) {
+    TORCH_CHECK(part.has_value() && part->is_cuda() && part->scalar_type() == at::kFloat && part->is_contiguous() &&
+                part->numel() >= B * H * Z * 2 * (vdim + 2), "part must be f32 [B, H, Z, 2, vdim + 2]");
+    pp = part->data_ptr<float>();
+  }
+  long gs = 0;
+  const void* gp = gate_rows(gate, q, gate_col, H * vdim, &gs);
+  CHECK_RC(lk_diff_attention_decode(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), ip(bt), (int)bt.stride(0), ip(ctx), (int)B, (int)Z,
+                                    (int)H, (int)G, (int)dim, (int)vdim, (int)kc.size(2), (float)scale, (float)tcoef, (int)tevery,
+                                    fp(lam, 1, "lam"), (float)eps, (int)norm_vdim, (float)oscale, gp, gs, (int)gate_col, out.data_ptr(),
+                                    out.stride(0), pp, esz_of(q, "q"), cur_stream()), "diff_attention_decode");
+}
+
+void tile_attention_prefill(const at::Tensor& q, const at::Tensor& kc, const at::Tensor& vc, const at::Tensor& bt, const at::Tensor& cu_q,
+                            const at::Tensor& ctx, const at::Tensor& ts, const at::Tensor& tq, int64_t maps, int64_t H, int64_t G, int64_t dim,
+                            int64_t vdim, double scale, double cap, double tcoef, int64_t tevery, const c10::optional<at::Tensor>& lam, double eps,
+                            int64_t norm_vdim, double oscale, const at::Tensor& gate, int64_t gate_col, at::Tensor& out) {
+  TORCH_CHECK(maps == 1 || maps == 2, "maps");
+  check_diff_inputs(q, kc, vc, bt, ctx, maps, H, G, dim, vdim, out);
+  CHECK_BF16(q);
+  check_tiles(bt, cu_q, ctx, ts, tq);
+  long gs = 0;
+  const void* gp = gate_rows(gate, q, gate_col, H * vdim, &gs);
+  CHECK_RC(lk_tile_attention_prefill(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), ip(bt), (int)bt.stride(0), ip(cu_q), ip(ctx), ip(ts),
+                                     ip(tq), (int)ts.numel(), (int)maps, (int)H, (int)G, (int)dim, (int)vdim, (int)kc.size(2), (float)scale,
+                                     (float)cap, (float)tcoef, (int)tevery, fpo(lam, 1, "lam"), (float)eps, (int)norm_vdim, (float)oscale, gp, gs,
+                                     (int)gate_col, out.data_ptr(), out.stride(0), cur_stream()), "tile_attention_prefill");
+}
+
+void head_delta(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, const at::Tensor& b, const at::Tensor& a, const at::Tensor& dt_bias,
+                const at::Tensor& A_log, const at::Tensor& gate, const at::Tensor& norm_w, double eps, at::Tensor& state, const at::Tensor& cu,
+                const at::Tensor& slots, const at::Tensor& positions, int64_t H, int64_t Hk, int64_t dk, int64_t dv, at::Tensor& out,
+                int64_t max_len) {
+  const int esz = esz_of(q, "q");
+  const long T = q.size(0);
+  TORCH_CHECK(H >= 1 && Hk >= 1 && H % Hk == 0 && dk >= 1 && dk <= 256 && dv >= 1 && dv <= 1024 && max_len >= 1, "head_delta sizes");
+  CHECK_CUDA(q); CHECK_LASTDIM(q);
+  TORCH_CHECK(q.dim() == 2 && q.size(1) >= Hk * dk, "q shape");
+  check_rows(k, T, Hk * dk, "k"); check_rows(v, T, H * dv, "v"); check_rows(b, T, H, "b"); check_rows(a, T, H, "a");
+  check_rows(gate, T, H * dv, "gate"); check_rows(out, T, H * dv, "out");
+  for (const at::Tensor* t : {&k, &v, &b, &a, &gate, static_cast<const at::Tensor*>(&out)}) same_type(*t, q, "operands");
+  CHECK_CUDA(state); CHECK_F32(state); CHECK_CONTIG(state);
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == dk && state.size(3) == dv, "state must be [slots, H, dk, dv]");
+  CHECK_CUDA(cu); CHECK_I32(cu); CHECK_CONTIG(cu); CHECK_CUDA(slots); CHECK_I32(slots); CHECK_CONTIG(slots); CHECK_CUDA(positions);
+  CHECK_I32(positions); CHECK_CONTIG(positions);
+  const long S = cu.numel() - 1;
+  TORCH_CHECK(S >= 0 && slots.numel() >= S && positions.numel() >= T, "sequences");
+  at::Tensor pre, o;
+  if (max_len > 1) {
+    pre = at::empty({T, H, lk_head_delta_pre()}, state.options());
+    o = at::empty({T, H * dv}, state.options());
+  }
+  CHECK_RC(lk_head_delta(q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), b.data_ptr(), b.stride(0), a.data_ptr(),
+                         a.stride(0), fp(dt_bias, H, "dt_bias"), fp(A_log, H, "A_log"), gate.data_ptr(), gate.stride(0),
+                         fp(norm_w, H * dv, "norm_w"), (float)eps, state.data_ptr<float>(), ip(cu), ip(slots), ip(positions), (int)S, T, (int)H,
+                         (int)Hk, (int)dk, (int)dv, out.data_ptr(), out.stride(0), (int)max_len, max_len > 1 ? pre.data_ptr<float>() : nullptr,
+                         max_len > 1 ? o.data_ptr<float>() : nullptr, esz, cur_stream()), "head_delta");
+}
+
 at::Tensor mlstm_scan(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, const at::Tensor& gates, at::Tensor& S, at::Tensor& nm,
                       const at::Tensor& cu, const at::Tensor& slots, const at::Tensor& positions, int64_t H, int64_t dk, int64_t dv, double q_scale,
                       int64_t max_len) {
@@ -1977,6 +2125,12 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gate_proj", &gate_proj);
   m.def("router_choice", &router_choice);
   m.def("mlstm_scan", &mlstm_scan);
+  m.def("stream_sandwich_layernorm", &stream_sandwich_layernorm);
+  m.def("qkv_file", &qkv_file);
+  m.def("diff_attention_prefill", &diff_attention_prefill);
+  m.def("diff_attention_decode", &diff_attention_decode);
+  m.def("tile_attention_prefill", &tile_attention_prefill);
+  m.def("head_delta", &head_delta);
   m.def("head_linear", &head_linear);
   m.def("latent_attn_prefill", &latent_attn_prefill);
   m.def("latent_attn_decode", &latent_attn_decode);

@@ -295,11 +295,11 @@ int lk_normrope_kv_write(void* qkv, long qs, long T, int H, int G, int dim, int 
 int lk_sinkattn_prefill(const void* q, long qs, const void* kc, const void* vc, const int* bt, int bt_stride, const int* cu_q,
                         const int* ctx_lens, const int* tile_seq, const int* tile_q0, int ntiles, int H, int G, int dim, int vdim,
                         int BS, const float* hscale, int mkind, int msize, int sink, const void* gate, long gs, int gcol, void* out,
-                        long os, const void* pkc, const void* pvc, int pool, int keep, float cap, int gelem, int esz, hipStream_t st);
+                        long os, const void* pkc, const void* pvc, int pool, int keep, float cap, int gelem, float oscale, int esz, hipStream_t st);
 int lk_sinkattn_decode(const void* q, long qs, const void* kc, const void* vc, const int* bt, int bt_stride, const int* ctx_lens,
                        int B, int Z, int H, int G, int dim, int vdim, int BS, const float* hscale, int mkind, int msize, int sink,
                        const void* gate, long gs, int gcol, void* out, long os, float* part, const void* pkc, const void* pvc,
-                       int pool, int keep, float cap, int gelem, int esz, hipStream_t st);
+                       int pool, int keep, float cap, int gelem, float oscale, int esz, hipStream_t st);
 
 // csrc/window_ops.hip: gated + normed sublayer result into the f32 stream (+ the next norm), RMS norm of a column block,
 // pair rotation + key assembly + paged K / V write, pooled (mean) keys / values of finished blocks
@@ -343,6 +343,30 @@ int lk_gate_proj(const void* h, long hs, const void* w, const float* bias, int N
 int lk_router_choice(const void* h, long hs, const void* w, int E, int K, long rows, int top, int groups, int keep, float scale, int score,
                      const float* corr, int gscore, int* experts, float* weights, int esz, hipStream_t st);
 
+// causal attention with biased projections and element gates (qkv_file.hip, attn_diff.hip, attn_tile.hip), gated delta rule with one
+// decay per head (head_delta.hip), stream normed in front of and behind every sublayer (stream_ln.hip)
+int lk_stream_sandwich(float* x, const void* y, long ys, int y_esz, const float* wp, const float* bp, const float* add, const float* w,
+                       const float* b, float eps, const long* idx, long rows, void* out, long os, int out_esz, int W, hipStream_t st);
+int lk_qkv_file(void* u, long us, long T, int H, int G, int dim, int vdim, const float* bias, const float* qw, const float* kw, int norm_q,
+                int norm_k, float eps, int rot, const float* freq, float mag, const int* positions, void* kc, void* vc, const int* slots,
+                int BS, int esz, hipStream_t st);
+int lk_diff_attention_prefill(const void* q, long qs, const void* kc, const void* vc, const int* bt, int bt_stride, const int* cu_q,
+                              const int* ctx_lens, const int* tile_seq, const int* tile_q0, int ntiles, int H, int G, int dim, int vdim,
+                              int BS, float scale, float tcoef, int tevery, const float* lam, float eps, int norm_vdim, float oscale,
+                              const void* gate, long gs, int gcol, void* out, long os, int esz, hipStream_t st);
+int lk_diff_attention_decode(const void* q, long qs, const void* kc, const void* vc, const int* bt, int bt_stride, const int* ctx_lens, int B,
+                             int Z, int H, int G, int dim, int vdim, int BS, float scale, float tcoef, int tevery, const float* lam, float eps,
+                             int norm_vdim, float oscale, const void* gate, long gs, int gcol, void* out, long os, float* part, int esz,
+                             hipStream_t st);
+int lk_tile_attention_prefill(const void* q, long qs, const void* kc, const void* vc, const int* bt, int bt_stride, const int* cu_q,
+                              const int* ctx_lens, const int* tile_seq, const int* tile_q0, int ntiles, int maps, int H, int G, int dim,
+                              int vdim, int BS, float scale, float cap, float tcoef, int tevery, const float* lam, float eps, int norm_vdim,
+                              float oscale, const void* gate, long gs, int gcol, void* out, long os, hipStream_t st);
+int lk_head_delta_pre();
+int lk_head_delta(const void* q, long qs, const void* k, long ks, const void* v, long vs, const void* b, long bs, const void* a, long as,
+                  const float* dt_bias, const float* A_log, const void* gate, long gs, const float* norm_w, float eps, float* state,
+                  const int* cu, const int* slots, const int* positions, int S, long T, int H, int Hk, int dk, int dv, void* out, long os,
+                  int max_len, float* pre, float* o, int esz, hipStream_t st);
 // csrc/mlstm.hip: matrix memory with exponential gates (S [slots, H, dk, dv], n | m [slots, H, ceil(dv / 64), dk + 4])
 int lk_mlstm_scan(const void* q, long qs, const void* k, long ks, const void* v, long vs, int esz, const float* gates, long gs, float q_scale,
                   float* S, float* nm, const int* cu, const int* slots, const int* positions, int seqs, int H, int dk, int dv, float* o,

@@ -130,6 +130,116 @@ __global__ __launch_bounds__(256) void stream_layernorm_kernel(float* __restrict
   }
 }
 
+// A sublayer boundary of a stream normed in front and behind:  x <- x + LN(y) wp + bp [+ add],  out = LN(x) w + b, the row in registers
+// between the four reductions.  One workgroup per output row, columns as in the kernel above.
+//   idx == null: x is updated in place;  idx != null: row idx[r] of x and y is read, nothing of x is written.
+template <typename TY, typename TO, int MAXI, int V>
+__global__ __launch_bounds__(256) void stream_sandwich_kernel(float* __restrict__ x, const TY* __restrict__ y, long ys,
+                                                              const float* __restrict__ wp, const float* __restrict__ bp,
+                                                              const float* __restrict__ add, const float* __restrict__ w,
+                                                              const float* __restrict__ b, float eps, const long* __restrict__ idx,
+                                                              TO* __restrict__ out, long os, int W) {
+  __shared__ float red[4];
+  const long orow = blockIdx.x, row = idx ? idx[orow] : orow;
+  const int ng = W / V;   // column groups (W % V == 0)
+  float v[MAXI][V], xr[MAXI][V];
+  auto ldn = [](const auto* p, float (&f)[V]) {
+    using E = std::remove_cv_t<std::remove_reference_t<decltype(*p)>>;
+    if constexpr (V == 4 && sizeof(E) == 4) {
+      const floatx4 t = *reinterpret_cast<const floatx4*>(p);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) f[e] = t[e];
+    } else if constexpr (V == 4) {
+      const short4_t t = *reinterpret_cast<const short4_t*>(p);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) f[e] = bf2f((bf16_t)t[e]);
+    } else {
+      f[0] = ldv<E>(p);
+    }
+  };
+  // v becomes (v - mean) * rsqrt(var + eps); columns past W hold zeros
+  auto norm = [&]() {
+    float s = 0.f;
+#pragma unroll
+    for (int i = 0; i < MAXI; ++i)
+#pragma unroll
+      for (int e = 0; e < V; ++e) s += v[i][e];
+    const float mean = block_sum<4>(s, red) / (float)W;
+    float q = 0.f;
+#pragma unroll
+    for (int i = 0; i < MAXI; ++i)
+      if ((int)threadIdx.x + 256 * i < ng) {
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+          v[i][e] -= mean;
+          q += v[i][e] * v[i][e];
+        }
+      }
+    const float inv = 1.f / sqrtf(block_sum<4>(q, red) / (float)W + eps);
+#pragma unroll
+    for (int i = 0; i < MAXI; ++i)
+#pragma unroll
+      for (int e = 0; e < V; ++e) v[i][e] *= inv;
+  };
+#pragma unroll
+  for (int i = 0; i < MAXI; ++i) {
+    const int c = (threadIdx.x + 256 * i) * V;
+#pragma unroll
+    for (int e = 0; e < V; ++e) v[i][e] = xr[i][e] = 0.f;
+    if ((int)threadIdx.x + 256 * i < ng) {
+      ldn(x + row * W + c, xr[i]);
+      if (y) ldn(y + row * ys + c, v[i]);
+    }
+  }
+  if (y) norm();
+#pragma unroll
+  for (int i = 0; i < MAXI; ++i) {
+    const int c = (threadIdx.x + 256 * i) * V;
+    if ((int)threadIdx.x + 256 * i < ng) {
+      float ww[V], bb[V];
+      if (y) {
+        ldn(wp + c, ww);
+        ldn(bp + c, bb);
+#pragma unroll
+        for (int e = 0; e < V; ++e) xr[i][e] += v[i][e] * ww[e] + bb[e];
+      }
+      if (add) {
+        ldn(add + c, ww);
+#pragma unroll
+        for (int e = 0; e < V; ++e) xr[i][e] += ww[e];
+      }
+      if (!idx && (y || add)) {
+        if constexpr (V == 4) *reinterpret_cast<floatx4*>(x + row * W + c) = floatx4{xr[i][0], xr[i][1], xr[i][2], xr[i][3]};
+        else x[row * W + c] = xr[i][0];
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < V; ++e) v[i][e] = xr[i][e];
+  }
+  norm();
+#pragma unroll
+  for (int i = 0; i < MAXI; ++i) {
+    const int c = (threadIdx.x + 256 * i) * V;
+    if ((int)threadIdx.x + 256 * i < ng) {
+      float ww[V], bb[V], r[V];
+      ldn(w + c, ww);
+      ldn(b + c, bb);
+#pragma unroll
+      for (int e = 0; e < V; ++e) r[e] = v[i][e] * ww[e] + bb[e];
+      if constexpr (V == 4 && sizeof(TO) == 4) {
+        *reinterpret_cast<floatx4*>(out + orow * os + c) = floatx4{r[0], r[1], r[2], r[3]};
+      } else if constexpr (V == 4) {
+        short4_t t;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) t[e] = (short)f2bf(r[e]);
+        *reinterpret_cast<short4_t*>(out + orow * os + c) = t;
+      } else {
+        stv<TO>(out + orow * os + c, r[0]);
+      }
+    }
+  }
+}
+
 template <typename T, bool EXACT>
 __global__ __launch_bounds__(256) void gelu_tanh_mul_kernel(const T* __restrict__ gu, long gs, T* __restrict__ out, long os, int F) {
   const long t = blockIdx.x;
@@ -188,6 +298,31 @@ int launch_ln(float* x, const void* y, long ys, const float* ls, float alpha, co
   return 0;
 }
 
+template <typename TY, typename TO>
+int launch_sandwich(float* x, const void* y, long ys, const float* wp, const float* bp, const float* add, const float* w, const float* b,
+                    float eps, const long* idx, void* out, long os, long rows, int W, hipStream_t st) {
+  const auto a16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };   // (a null pointer passes)
+  const bool vec = W % 4 == 0 && ys % 4 == 0 && os % 4 == 0 && a16(y) && a16(out) && a16(x) && a16(wp) && a16(bp) && a16(add) && a16(w) && a16(b);
+#define LK_SW(MAXI, V)                                                                                                       \
+  stream_sandwich_kernel<TY, TO, MAXI, V><<<(unsigned)rows, 256, 0, st>>>(x, (const TY*)y, ys, wp, bp, add, w, b, eps, idx, \
+                                                                          (TO*)out, os, W)
+  if (vec) {
+    if (W <= 1024) LK_SW(1, 4);
+    else if (W <= 2048) LK_SW(2, 4);
+    else if (W <= 4096) LK_SW(4, 4);
+    else if (W <= 16384) LK_SW(16, 4);
+    else return -1;
+  } else {
+    if (W <= 1024) LK_SW(4, 1);
+    else if (W <= 4096) LK_SW(16, 1);
+    else if (W <= 16384) LK_SW(64, 1);
+    else return -1;
+  }
+#undef LK_SW
+  LK_CHECK_LAUNCH();
+  return 0;
+}
+
 }  // namespace
 
 int lk_embed_stream(const int* ids, const void* tok, long V, long T, int W, float* x, void* copy, float scale, int esz,
@@ -209,6 +344,18 @@ int lk_stream_layernorm(float* x, const void* y, long ys, int y_esz, const float
   if (yb) return launch_ln<bf16_t, float>(x, y, ys, ls, alpha, w, b, eps, idx, out, os, rows, W, st);
   if (ob) return launch_ln<float, bf16_t>(x, y, ys, ls, alpha, w, b, eps, idx, out, os, rows, W, st);
   return launch_ln<float, float>(x, y, ys, ls, alpha, w, b, eps, idx, out, os, rows, W, st);
+}
+
+// x <- x + LN(y) wp + bp [+ add] (y, add may be null), out = LN(x) w + b; with idx x is only read
+int lk_stream_sandwich(float* x, const void* y, long ys, int y_esz, const float* wp, const float* bp, const float* add, const float* w,
+                       const float* b, float eps, const long* idx, long rows, void* out, long os, int out_esz, int W, hipStream_t st) {
+  if (rows <= 0) return 0;
+  if (!w || !b || !out || (y && (!wp || !bp))) return -1;
+  const bool yb = y && y_esz == 2, ob = out_esz == 2;
+  if (yb && ob) return launch_sandwich<bf16_t, bf16_t>(x, y, ys, wp, bp, add, w, b, eps, idx, out, os, rows, W, st);
+  if (yb) return launch_sandwich<bf16_t, float>(x, y, ys, wp, bp, add, w, b, eps, idx, out, os, rows, W, st);
+  if (ob) return launch_sandwich<float, bf16_t>(x, y, ys, wp, bp, add, w, b, eps, idx, out, os, rows, W, st);
+  return launch_sandwich<float, float>(x, y, ys, wp, bp, add, w, b, eps, idx, out, os, rows, W, st);
 }
 
 int lk_gelu_tanh_mul(const void* gu, long gs, void* out, long os, long rows, int F, int esz, hipStream_t st) {

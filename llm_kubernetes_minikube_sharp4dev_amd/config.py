@@ -133,6 +133,8 @@ class ModelPresets:
         "lumedra-1b": "lumedra-1b",
         "kafilorn-tiny": "kafilorn-tiny",
         "kafilorn-1b": "kafilorn-1b",
+        "kebepel-tiny": "kebepel-tiny",
+        "kebepel-1b": "kebepel-1b",
     })
     embedders: dict = field(default_factory=lambda: {
         "nomic-embed-text": "nomic-embed-text",

@@ -8,11 +8,12 @@ import torch
 
 from ..parallel.tp import SINGLE, TPGroup
 from .bert import EncoderModel
-from .configs import (DECODERS, ENCODERS, DecoderConfig, EncoderConfig, FusasunConfig, KafilornConfig, LebepelConfig, LumedraConfig, PemidraConfig, decoder_config,
-                      encoder_config)
+from .configs import (DECODERS, ENCODERS, DecoderConfig, EncoderConfig, FusasunConfig, KafilornConfig, KebepelConfig, LebepelConfig, LumedraConfig, PemidraConfig,
+                      decoder_config, encoder_config)
 from . import llama
 from .fusasun import FusasunModel
 from .kafilorn import KafilornModel
+from .kebepel import KebepelModel
 from .lebepel import LebepelModel
 from .llama import LlamaModel
 from .lumedra import LumedraModel
@@ -21,11 +22,11 @@ from .pemidra import PemidraModel, ranks_from_state_dict
 
 # decoder architectures by ``cfg.arch``
 DECODER_CLASSES = {"llama": LlamaModel, "opt": OPTModel, "lebepel": LebepelModel, "pemidra": PemidraModel,
-                   "fusasun": FusasunModel, "lumedra": LumedraModel, "kafilorn": KafilornModel}
+                   "fusasun": FusasunModel, "lumedra": LumedraModel, "kafilorn": KafilornModel, "kebepel": KebepelModel}
 # designs with a checkpoint format of their own (config.json read by ``<Config>.from_json``, tensors by
 # ``load_state_dict_native``)
 NATIVE_CONFIGS = {"lebepel": LebepelConfig, "pemidra": PemidraConfig, "fusasun": FusasunConfig, "lumedra": LumedraConfig,
-                  "kafilorn": KafilornConfig}
+                  "kafilorn": KafilornConfig, "kebepel": KebepelConfig}
 
 
 def _load_safetensors_dir(path: str) -> dict:
@@ -123,5 +124,5 @@ def build_encoder(name: str | EncoderConfig, device="cpu", dtype=torch.bfloat16,
 
 __all__ = ["build_decoder", "build_encoder", "load_decoder_dir", "checkpoint_architecture", "DECODER_CLASSES",
            "LebepelConfig", "LebepelModel", "PemidraConfig", "PemidraModel", "FusasunConfig", "FusasunModel", "LumedraConfig", "LumedraModel",
-           "KafilornConfig", "KafilornModel", "NATIVE_CONFIGS", "DECODERS", "ENCODERS", "DecoderConfig", "EncoderConfig",
+           "KafilornConfig", "KafilornModel", "KebepelConfig", "KebepelModel", "NATIVE_CONFIGS", "DECODERS", "ENCODERS", "DecoderConfig", "EncoderConfig",
            "LlamaModel", "OPTModel", "EncoderModel"]

@@ -93,6 +93,8 @@ class AttnMeta:
     max_seq_len: int = 1
     # sigmoid attention (sigmoid_paged_attention): its 16-query tile list, built once per step
     sig_tiles: Optional[tuple] = None
+    # staged prompt kernels (models/gated_attention.py): tile lists by queries per tile, built once per step
+    row_tiles: dict = field(default_factory=dict)
 
     @property
     def num_tokens(self) -> int:

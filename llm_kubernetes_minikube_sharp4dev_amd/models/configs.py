@@ -343,6 +343,95 @@ class KafilornConfig:
                            for l in self.layers]}
 
 
+@dataclass
+class KebepelConfig:
+    """The Kebepel design: sublayers with a layer norm (weight and bias) in front and one behind over an f32 residual stream,
+    differential attention layers and layers of row-normed attention beside a gated delta rule, a span of layers run ``loop_times``
+    times with shared weights (pass t adds a learned vector to the stream first, the first pass too; every pass has its
+    own caches and states).  Every size and constant comes from the checkpoint's ``config.json`` (:meth:`from_json`)."""
+    name: str
+    vocab_size: int
+    hidden: int
+    layers: list                 # [HybridLayer], type "attention" | "parallel"
+    norm_eps: float = 1e-5
+    loop_start: int = 0
+    loop_stop: int = 0
+    loop_times: int = 0          # 0: no loop (no step vectors)
+    max_position: int = 1 << 20  # nothing in the design bounds a sequence; engines pass their own limit
+    arch: str = "kebepel"
+    bos_token_id: int = 0
+    eos_token_ids: tuple = ()
+    tie_word_embeddings: bool = False
+
+    MIXERS = ("attention", "parallel")
+
+    def __post_init__(self):
+        for l in self.layers:
+            if l.type not in self.MIXERS:
+                raise ValueError(f"unknown mixer type {l.type!r}")
+            if l.mlp is not None and l.mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"unknown feed-forward kind {l.mlp.get('kind')!r}")
+        self.layer_runs()
+
+    def layer_runs(self) -> list:
+        """[(layer index, pass whose step vector is added first or None)] in execution order: the looped span is
+        unrolled; every run has a cache or state of its own."""
+        n = len(self.layers)
+        a, b, t = self.loop_start, self.loop_stop, self.loop_times
+        if t == 0:
+            return [(i, None) for i in range(n)]
+        if not (0 <= a < b <= n) or t < 1:
+            raise ValueError(f"loop [{a}, {b}) x {t} does not fit {n} layers")
+        runs = [(i, None) for i in range(a)]
+        for k in range(t):
+            runs += [(i, k if i == a else None) for i in range(a, b)]
+        return runs + [(i, None) for i in range(b, n)]
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layer_runs())
+
+    @classmethod
+    def from_json(cls, d: dict, name: str = "kebepel") -> "KebepelConfig":
+        layers = [HybridLayer(l["type"], dict(l["mixer"]), dict(l["mlp"]) if l.get("mlp") else None)
+                  for l in d["layers"]]
+        loop = d.get("loop") or {}
+        return cls(name=name, vocab_size=int(d["vocab"]), hidden=int(d["width"]), layers=layers,
+                   norm_eps=float((d.get("norm") or {}).get("eps", 1e-5)), loop_start=int(loop.get("start", 0)),
+                   loop_stop=int(loop.get("stop", 0)), loop_times=int(loop.get("times", 0)),
+                   max_position=int(d.get("max_positions", 1 << 20)))
+
+    def to_json(self) -> dict:
+        d = {"architecture": "Kebepel", "vocab": self.vocab_size, "width": self.hidden, "norm": {"eps": self.norm_eps},
+             "layers": [{"type": l.type, "mixer": dict(l.mixer), "mlp": dict(l.mlp) if l.mlp else None} for l in self.layers]}
+        if self.loop_times:
+            d["loop"] = {"start": self.loop_start, "stop": self.loop_stop, "times": self.loop_times}
+        return d
+
+
+def kebepel_layers(n: int, heads: int, head_dim: int, ff: int, kv_heads: Optional[int] = None, rot_dims: Optional[int] = None,
+                   conv: int = 4, diff: float = 0.3, softcap: float = 50.0, original: int = 8192, temp_every: int = 4096,
+                   pattern=("attention", "parallel")) -> list:
+    """``n`` layers cycling through ``pattern`` with one set of head sizes (presets and benchmarks); a differential head's two
+    maps share ``head_dim`` query / key columns."""
+    kv = kv_heads or heads
+    out = []
+    for i in range(n):
+        t = pattern[i % len(pattern)]
+        if t == "attention":
+            d = head_dim // 2
+            mixer = {"heads": heads, "kv_heads": kv, "dim": d, "vdim": head_dim, "scale": d ** -0.5, "diff": diff,
+                     "q_temp": {"coef": 0.1, "every": temp_every}}
+        else:
+            mixer = {"left": {"heads": heads, "kv_heads": kv, "dim": head_dim, "vdim": head_dim, "scale": head_dim ** -0.5, "softcap": softcap,
+                              "rot": {"base": 500000.0, "dims": rot_dims or head_dim,
+                                      "scaling": {"factor": 8.0, "original": original, "fast": 32.0, "slow": 1.0}}},
+                     "right": {"heads": heads, "kv_heads": heads, "dim": head_dim, "vdim": head_dim, "conv": conv},
+                     "left_scale": 0.8, "right_scale": 1.1}
+        out.append(HybridLayer(t, mixer, {"kind": "dense", "ff": ff} if ff else None))
+    return out
+
+
 def kafilorn_layers(n: int, heads: int, head_dim: int, dense_ff: int, expert_ff: int = 0, experts: int = 0, top: int = 2,
                     window: int = 1024, rot_dim: int = 64, q_rank: int = 768, kv_rank: int = 512, groups: int = 4, keep: int = 2,
                     shared_ff: int = 0, gate_cap: float = 15.0, pattern=("mlstm", "latent_attention", "shared_latent")) -> list:
@@ -533,6 +622,14 @@ DECODERS.update({
                                                                               shared_ff=1408), streams=4),
 })
 
+DECODERS.update({
+    # differential attention layers and parallel row-normed attention / gated delta rule layers, a looped span (random-init presets)
+    "kebepel-tiny": KebepelConfig("kebepel-tiny", 32768, 128, kebepel_layers(3, 4, 24, 80, kv_heads=2, rot_dims=16, conv=3, original=64,
+                                                                              temp_every=32), loop_start=1, loop_stop=3, loop_times=2),
+    "kebepel-1b": KebepelConfig("kebepel-1b", 32768, 2048, kebepel_layers(16, 16, 128, 5632, kv_heads=4), loop_start=4, loop_stop=12,
+                                loop_times=2),
+})
+
 ENCODERS = {
     "bge-base": EncoderConfig("bge-base", "bert", 12, 768, 12, 3072, 30522, pooling="cls"),
     "minilm-l6": EncoderConfig("minilm-l6", "bert", 6, 384, 12, 1536, 30522, pooling="mean"),
@@ -560,6 +657,22 @@ def encoder_config(name: str, **overrides) -> EncoderConfig:
 
 
 def param_count(cfg) -> int:
+    if isinstance(cfg, KebepelConfig):
+        W = cfg.hidden
+        n = (2 * cfg.vocab_size + 2 + cfg.loop_times) * W
+        for l in cfg.layers:
+            m = l.mixer
+            if l.type == "attention":
+                qk = 2 * (m["heads"] + m["kv_heads"]) * m["dim"] + m["kv_heads"] * m["vdim"]
+                n += qk * (W + 1) + 2 * W * m["heads"] * m["vdim"] + 4 * m["dim"]
+            else:
+                a, b = m["left"], m["right"]
+                qk = (a["heads"] + a["kv_heads"]) * a["dim"]
+                n += (qk + a["kv_heads"] * a["vdim"]) * (W + 1) + qk + 2 * W * a["heads"] * a["vdim"]
+                conv = 2 * b["kv_heads"] * b["dim"] + b["heads"] * b["vdim"]
+                n += conv * (W + b["conv"]) + 2 * b["heads"] * (W + 1) + 2 * W * b["heads"] * b["vdim"] + b["vdim"]
+            n += 4 * W + ((3 * l.mlp["ff"] + 4) * W if l.mlp else 0)
+        return n
     if isinstance(cfg, KafilornConfig):
         W, S = cfg.hidden, cfg.streams
         n = 2 * cfg.vocab_size * W + W

@@ -6,7 +6,9 @@ q, k, v) and the generalized delta rule.  All but the first are members of
     S_t = diag(w_t) S_(t-1) - p_t (z_t^T S_(t-1)) + k_t v_t^T,    o_t = S_t^T q_t
 
 and share one scan kernel (``ops.delta_scan``); what differs is how the f32 operands are made from the
-layer's projections.  A mixer layer owns one f32 state tensor ``[slots, H, dk, dv]`` (and, with
+layer's projections.  The gated delta rule with one decay per head (``head_delta_mixer``) has kernels of its own beside the scan:
+a constant decay over the key channels makes prompt portions masked products per chunk of tokens (``ops.head_delta``).
+A mixer layer owns one f32 state tensor ``[slots, H, dk, dv]`` (and, with
 convolutions, their last ``taps - 1`` inputs), one row per state slot
 (``engine.block_manager.StateSlotPool``); a step's sequences -- prompt portions of any length and
 one-token decode rows alike -- are described by ``AttnMeta.seq_cu`` / ``state_slots``, and a sequence whose
@@ -263,3 +265,52 @@ def gated_delta_mixer(h, w_in, rows: FusedRows, conv_w, a2, dt_bias, A_log, g2, 
                        spec.vdim, max_len=meta.max_seq_len)
     y = ops.head_norm_gate(o, graw, norm_w, spec.heads, eps, ops.GATE_SIGMOID, out_dtype)
     return ops.linear(y, w_out)
+
+
+@dataclass
+class HeadDeltaSpec:
+    """Gated delta rule with one decay per head and token: ``S <- g S; S <- S + k (beta (v - S^T k))^T; o = S^T q`` on unit q, k
+    (after causal convolutions and SiLU on q, k, v), ``beta = sigmoid(b)``, ``g = exp(-exp(A_log) softplus(a + dt_bias))`` with a, b
+    projections of one column per head; each head's o RMS-normed, times a weight shared by the heads, times silu(W_g h)."""
+    heads: int
+    kv_heads: int      # q / k heads (value head h reads q / k head h // (heads / kv_heads))
+    dim: int
+    vdim: int
+    conv: int          # taps of the causal convolutions on q, k and v
+
+    @classmethod
+    def from_dict(cls, m: dict) -> "HeadDeltaSpec":
+        s = cls(int(m["heads"]), int(m.get("kv_heads", m["heads"])), int(m["dim"]), int(m.get("vdim", m["dim"])), int(m.get("conv", 4)))
+        if s.heads % s.kv_heads or not 1 <= s.conv <= 8 or not ops.head_delta_supported(s.dim, s.vdim):
+            raise ValueError(f"unsupported gated delta-rule sizes {m}")
+        return s
+
+    def segments(self) -> list:
+        """Column blocks of the input projection, q | k | v first and adjacent (the convolution runs over them)."""
+        return [("dq", self.kv_heads * self.dim), ("dk", self.kv_heads * self.dim), ("dv", self.heads * self.vdim), ("db", self.heads),
+                ("da", self.heads), ("dg", self.heads * self.vdim)]
+
+    def conv_rows(self) -> FusedRows:
+        """The convolution's own column layout (offsets from the first q column)."""
+        return FusedRows(self.segments()[:3])
+
+    def make_state(self, slots: int, dtype, device):
+        """(conv state [slots, taps - 1, C] in the activation dtype, S f32 [slots, heads, dim, vdim])."""
+        return (torch.zeros(slots, max(self.conv - 1, 1), self.conv_rows().total, dtype=dtype, device=device),
+                torch.zeros(slots, self.heads, self.dim, self.vdim, dtype=torch.float32, device=device))
+
+    def state_bytes(self, dtype) -> int:
+        esz = torch.tensor([], dtype=dtype).element_size()
+        return max(self.conv - 1, 1) * self.conv_rows().total * esz + self.heads * self.dim * self.vdim * 4
+
+
+def head_delta_mixer(u, rows: FusedRows, conv_rows: FusedRows, conv_w, dt_bias, A_log, norm_w, spec: HeadDeltaSpec, eps: float, state, meta, out):
+    """u [T, .. | dq | dk | dv | db | da | dg]: a fused projection that holds this mixer's columns (``rows``).  Causal conv + SiLU
+    over q | k | v, then unit norms, gates, the recurrence, head norm and gate (``ops.head_delta``) into ``out`` [T, >= heads *
+    vdim] (the output projection is the caller's: its weight may be shared with a mixer beside this one, and a scale of the
+    result belongs in ``norm_w``).  ``state`` = (conv, S) of this layer."""
+    conv_state, S = state
+    xc = ops.conv_silu(u, rows.off["dq"], conv_rows.total, conv_w, None, conv_state, meta.seq_cu, meta.state_slots, meta.positions, meta.max_seq_len)
+    return ops.head_delta(conv_rows.cols(xc, "dq"), conv_rows.cols(xc, "dk"), conv_rows.cols(xc, "dv"), rows.cols(u, "db"), rows.cols(u, "da"),
+                          dt_bias, A_log, rows.cols(u, "dg"), norm_w, eps, S, meta.seq_cu, meta.state_slots, meta.positions, spec.heads,
+                          spec.kv_heads, spec.dim, spec.vdim, out, max_len=meta.max_seq_len)

@@ -19,13 +19,16 @@ from .mixers import (conv_silu, embed_pos, gated_group_rmsnorm, linear_swiglu_an
                      sig_prefill_tiles, sigattn_supported, sigmoid_attention_decode, sigmoid_attention_prefill,
                      softcap, ssm_scan, stream_rmsnorm, unitnorm_kv_write, embed_stream, stream_layernorm, gelu_tanh_mul,
                      dual_rmsnorm_mean, normrope_kv_write, sink_attention_prefill, sink_attention_decode, mask_first_key,
-                     pooled_blocks_seen, MASK_CAUSAL, MASK_CHUNK, MASK_WINDOW)
+                     pooled_blocks_seen, stream_sandwich_layernorm, MASK_CAUSAL, MASK_CHUNK, MASK_WINDOW, SIG_TILE_ROWS)
 from .window import moe_route, pool_kv_write, rms_cols, rot_kv_write, run_experts, stream_gated_norm, table_experts  # noqa: F401
 from .routed import clamped_glu, routed_experts, router_topk, sigmoid_mul_, silu_, stream_parallel_norm  # noqa: F401
 from .hyper import (GROUP_MAX, GROUP_TOP2, MAX_STREAMS, SCORE_SIGMOID, SCORE_SOFTMAX, gate_proj, relu_sq_, router_choice,  # noqa: F401
                     stream_hyper_norm)
 from .latent import (head_linear, latent_attention_decode, latent_attention_prefill, latent_decode_splits, latent_prep,  # noqa: F401
                      latent_query_rot, latent_row)
+from .diff import (diff_attention_decode, diff_attention_prefill, diff_attention_supported, diff_prefill_rows, qkv_file, row_tiles,  # noqa: F401
+                   tile_attention_prefill, tile_attention_rows, tile_attention_supported)
+from .head_delta import head_delta, head_delta_supported  # noqa: F401
 from .mlstm import mlstm_scan, mlstm_state, mlstm_supported  # noqa: F401
 from .delta import (delta_scan, delta_scan_supported, gated_delta_prep, general_delta_prep, head_norm_gate, tanh_,  # noqa: F401
                     GATE_SIGMOID, GATE_SILU)

@@ -24,7 +24,7 @@ from ._ext import lib, use_hip
 
 __all__ = ["embed_pos", "stream_rmsnorm", "softcap", "linear_swiglu_any", "unitnorm_kv_write", "sig_prefill_tiles", "sig_decode_splits",
            "sigmoid_attention_prefill", "sigmoid_attention_decode", "sigattn_supported", "conv_silu", "ssm_scan",
-           "gated_group_rmsnorm", "embed_stream", "stream_layernorm", "gelu_tanh_mul", "dual_rmsnorm_mean", "normrope_kv_write",
+           "gated_group_rmsnorm", "embed_stream", "stream_layernorm", "stream_sandwich_layernorm", "gelu_tanh_mul", "dual_rmsnorm_mean", "normrope_kv_write",
            "sink_attention_prefill", "sink_attention_decode", "mask_first_key", "pooled_blocks_seen", "MASK_CAUSAL", "MASK_CHUNK",
            "MASK_WINDOW"]
 
@@ -314,6 +314,28 @@ def stream_layernorm(x, y, ls, alpha: float, w, b, eps: float, out_dtype=torch.b
     return x if out_dtype == torch.float32 else x.to(out_dtype)
 
 
+def stream_sandwich_layernorm(x, y, w_post, b_post, add, w_next, b_next, eps: float, out_dtype=torch.bfloat16, idx=None):
+    """One sublayer boundary of a stream whose sublayers are normed in front and behind: ``x += LN(y) w_post + b_post`` (``y`` None:
+    nothing), ``x += add`` (f32 [W], a vector added to every row; None: nothing), both in place in f32, then ``LN(x) w_next + b_next``
+    in ``out_dtype``.  LN(v) = (v - mean) / sqrt(mean squared deviation + eps).  With ``idx`` (int64 rows) only those rows are computed
+    and ``x`` is left as it was (the rows that feed the LM head)."""
+    if use_hip(x):
+        return lib().stream_sandwich_layernorm(x, y, w_post, b_post, add, w_next, b_next, float(eps), idx, out_dtype)
+
+    def ln(v, w, b):
+        d = v - v.mean(-1, keepdim=True)
+        return d / torch.sqrt(d.pow(2).mean(-1, keepdim=True) + eps) * w + b
+
+    v = x if idx is None else x.index_select(0, idx)
+    if y is not None:
+        v = v + ln((y if idx is None else y.index_select(0, idx)).float(), w_post, b_post)
+    if add is not None:
+        v = v + add
+    if idx is None and v is not x:
+        x.copy_(v)
+    return ln(v, w_next, b_next).to(out_dtype)
+
+
 def gelu_tanh_mul(gu):
     """[T, 2F] = [gate | up] -> gelu_tanh(gate) * up, [T, F] in the same dtype."""
     if use_hip(gu):
@@ -471,7 +493,7 @@ def _gated(o, gate, r0, r1, gate_col, H, vdim, gate_elem):
 
 def sink_attention_prefill(q, k_cache, v_cache, block_tables, cu_q, ctx_lens, H: int, G: int, dim: int, vdim: int, hscale,
                            mask_kind: int, mask_size: int, sink: bool, gate, gate_col: int, out, tiles=None, q_lens_cpu=None,
-                           pool=None, keep_first: int = 0, softcap: float = 0.0, gate_elem: bool = False):
+                           pool=None, keep_first: int = 0, softcap: float = 0.0, gate_elem: bool = False, out_scale: float = 1.0):
     """Softmax attention of query chunks over their sequences' cached keys inside the mask
     (``mask_first_key``), with ``sink``: one more term of score 0 and no value in the denominator.
     ``hscale`` f32 [H]: the score multiplier of each head.  ``gate`` (or None): rows aligned with ``q``
@@ -482,7 +504,7 @@ def sink_attention_prefill(q, k_cache, v_cache, block_tables, cu_q, ctx_lens, H:
     ``pool_kv_write`` at the logical position b of the same block table.
     ``keep_first`` (window masks, no pooling): positions below it stay visible to every later query.  ``softcap`` >
     0: a score s becomes softcap * tanh(s / softcap) before the softmax.  ``gate_elem``: the gate has one column
-    per output element, ``gate_col + h * vdim + d``, instead of one per head."""
+    per output element, ``gate_col + h * vdim + d``, instead of one per head.  ``out_scale``: the f32 result is multiplied by it."""
     _check_mask_options(mask_kind, pool, keep_first)
     if use_hip(q):
         if tiles is None:
@@ -492,7 +514,7 @@ def sink_attention_prefill(q, k_cache, v_cache, block_tables, cu_q, ctx_lens, H:
         pk, pv, P = pool if pool is not None else (None, None, 0)
         lib().sinkattn_prefill(q, k_cache, v_cache, block_tables, cu_q, ctx_lens, tiles[0], tiles[1], H, G, dim, vdim, hscale,
                                int(mask_kind), int(mask_size), bool(sink), gate, int(gate_col), out, pk, pv, int(P),
-                               int(keep_first), float(softcap), bool(gate_elem))
+                               int(keep_first), float(softcap), bool(gate_elem), float(out_scale))
         return out
     cu = cu_q.tolist()
     for b in range(len(cu) - 1):
@@ -502,13 +524,13 @@ def sink_attention_prefill(q, k_cache, v_cache, block_tables, cu_q, ctx_lens, H:
         qq = q[s0:s1, : H * dim].float().view(s1 - s0, H, dim)
         qpos = torch.arange(n - (s1 - s0), n, device=q.device)
         o = _sink_rows(qq, k, v, qpos, hscale, mask_kind, mask_size, sink, _pooled_of(pool, block_tables[b], n), keep_first, softcap)
-        out[s0:s1, : H * vdim] = _gated(o, gate, s0, s1, gate_col, H, vdim, gate_elem).reshape(s1 - s0, H * vdim).to(out.dtype)
+        out[s0:s1, : H * vdim] = (_gated(o, gate, s0, s1, gate_col, H, vdim, gate_elem) * out_scale).reshape(s1 - s0, H * vdim).to(out.dtype)
     return out
 
 
 def sink_attention_decode(q, k_cache, v_cache, block_tables, ctx_lens, H: int, G: int, dim: int, vdim: int, hscale,
                           mask_kind: int, mask_size: int, sink: bool, gate, gate_col: int, out, splits: int = 1, part=None,
-                          pool=None, keep_first: int = 0, softcap: float = 0.0, gate_elem: bool = False):
+                          pool=None, keep_first: int = 0, softcap: float = 0.0, gate_elem: bool = False, out_scale: float = 1.0):
     """One query row per sequence at its last position (ctx - 1) over its cached keys inside the mask
     (and the pooled blocks before it: see ``sink_attention_prefill``)."""
     B = q.shape[0]
@@ -519,7 +541,7 @@ def sink_attention_decode(q, k_cache, v_cache, block_tables, ctx_lens, H: int, G
         pk, pv, P = pool if pool is not None else (None, None, 0)
         lib().sinkattn_decode(q, k_cache, v_cache, block_tables, ctx_lens, int(splits), H, G, dim, vdim, hscale, int(mask_kind),
                               int(mask_size), bool(sink), gate, int(gate_col), out, part, pk, pv, int(P), int(keep_first),
-                              float(softcap), bool(gate_elem))
+                              float(softcap), bool(gate_elem), float(out_scale))
         return out
     for b in range(B):
         n = int(ctx_lens[b])
@@ -527,5 +549,5 @@ def sink_attention_decode(q, k_cache, v_cache, block_tables, ctx_lens, H: int, G
         qq = q[b:b + 1, : H * dim].float().view(1, H, dim)
         o = _sink_rows(qq, k, v, torch.tensor([n - 1], device=q.device), hscale, mask_kind, mask_size, sink,
                        _pooled_of(pool, block_tables[b], n), keep_first, softcap)
-        out[b:b + 1, : H * vdim] = _gated(o, gate, b, b + 1, gate_col, H, vdim, gate_elem).reshape(1, H * vdim).to(out.dtype)
+        out[b:b + 1, : H * vdim] = (_gated(o, gate, b, b + 1, gate_col, H, vdim, gate_elem) * out_scale).reshape(1, H * vdim).to(out.dtype)
     return out
