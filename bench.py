@@ -142,7 +142,8 @@ def parse():
     ap.add_argument("--json-out", default=None)
     ap.add_argument("--decoder-bench", action="store_true",
                     help="instead of the headline workload: prefill and decode tokens/s of the hybrid decoders "
-                         "(Lebepel by default; -- --models pemidra,lebepel,llama, fusasun,llama, lumedra,fusasun,llama or kafilorn,lumedra,llama for the others) beside a Llama decoder of "
+                         "(Lebepel by default; -- --models pemidra,lebepel,llama, fusasun,llama, lumedra,fusasun,llama, kafilorn,lumedra,llama or "
+                         "kebepel,pemidra,llama for the others) beside a Llama decoder of "
                          "equal size at a few layer sizes (benchmarks/decoder_bench.py; its own options follow after --)")
     args, rest = ap.parse_known_args()
     if rest and not args.decoder_bench:

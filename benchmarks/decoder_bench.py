@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Prefill and decode throughput of the hybrid decoders (Lebepel; Pemidra with ``--models pemidra,lebepel``;
 Fusasun with ``--models fusasun,llama``; Lumedra with ``--models lumedra,fusasun,llama``; Kafilorn with ``--models
-kafilorn,lumedra,llama``) beside a Llama decoder of the same width, depth, heads, head size, feed-forward and vocabulary (random
+kafilorn,lumedra,llama``; Kebepel with ``--models kebepel,pemidra,llama``) beside a Llama decoder of the same width, depth, heads, head size, feed-forward and vocabulary (random
 weights, bf16, one GPU), all through the same engine: prefill = S fresh prompts of L tokens in one step, decode = B sequences at
 context C, one token each per step (hipGraph replay).  ``bench.py --decoder-bench`` runs this.
 
@@ -33,9 +33,10 @@ VOCAB = 32768
 
 def models(width: int, which: str, device):
     from llm_kubernetes_minikube_sharp4dev_amd.models import build_decoder
-    from llm_kubernetes_minikube_sharp4dev_amd.models.configs import (FusasunConfig, KafilornConfig, LebepelConfig, LumedraConfig,
-                                                                      PemidraConfig, decoder_config, fusasun_layers, kafilorn_layers,
-                                                                      lebepel_layers, lumedra_layers, pemidra_layers)
+    from llm_kubernetes_minikube_sharp4dev_amd.models.configs import (FusasunConfig, KafilornConfig, KebepelConfig, LebepelConfig,
+                                                                      LumedraConfig, PemidraConfig, decoder_config, fusasun_layers,
+                                                                      kafilorn_layers, kebepel_layers, lebepel_layers, lumedra_layers,
+                                                                      pemidra_layers)
 
     L, H, G, D, FF, sh, sp, sn, sg = SIZES[width]
     if which == "lebepel":
@@ -70,6 +71,11 @@ def models(width: int, which: str, device):
         cfg = KafilornConfig(f"kafilorn-w{width}", VOCAB, width,
                              kafilorn_layers(L, H, D, FF * 3 // 2 // 256 * 256, FF // 4, 16, 2, window=512, rot_dim=64,
                                              q_rank=max(512, width // 2), kv_rank=512, groups=4, keep=2, shared_ff=FF // 2), streams=4)
+    elif which == "kebepel":
+        # differential attention (two maps of D / 2 per head on values of D) and causal row-normed attention with a score cap
+        # beside a gated delta rule (heads x D x D states) in turn, the same heads, kv heads and head size; every layer with the
+        # dense gated feed-forward; no looped span (a loop multiplies layer runs, not kernels)
+        cfg = KebepelConfig(f"kebepel-w{width}", VOCAB, width, kebepel_layers(L, H, D, FF, kv_heads=G))
     else:
         cfg = decoder_config("llama-3-8b", num_layers=L, hidden=width, num_heads=H, num_kv_heads=G, head_dim=D,
                              intermediate=FF, vocab_size=VOCAB, max_position=8192)
@@ -126,7 +132,7 @@ def run(width: int, which: str, a) -> dict:
 def main(argv=None):
     ap = argparse.ArgumentParser()
     ap.add_argument("--sizes", default="1024,2048,4096")
-    ap.add_argument("--models", default="lebepel,llama", help="comma list of lebepel, pemidra, fusasun, lumedra, kafilorn, llama")
+    ap.add_argument("--models", default="lebepel,llama", help="comma list of lebepel, pemidra, fusasun, lumedra, kafilorn, kebepel, llama")
     ap.add_argument("--prefill-seqs", type=int, default=4)
     ap.add_argument("--prefill-len", type=int, default=1024)
     ap.add_argument("--decode-batch", type=int, default=64)

@@ -74,42 +74,60 @@ LK_DEVICE void diff_run(const DiffParams& p, const QFrag<T, KP>& qf, int kvh, co
   const T* kc = reinterpret_cast<const T*>(p.kc);
   const T* vc = reinterpret_cast<const T*>(p.vc);
   const int krow = 8 * (n16 >> 2) + (n16 & 3);
-  for (int kb = k0 + 32 * step0; kb < k1; kb += 32 * stride) {
-    const T* kr[2];
+  // A step's page numbers are read two steps ahead and its K rows one step ahead, as soon as the products have consumed the current
+  // ones; its V rows before its own products: the loads of a step fly under the arithmetic of the one before.
+  int pk[2], pv;   // pages of the K rows / V columns of the next step to be requested
+  auto pages = [&](int kb) {
+#pragma unroll
+    for (int t = 0; t < 2; ++t) pk[t] = bt[min(kb + krow + 4 * t, k1 - 1) / p.BS];
+    pv = bt[min(kb + 8 * g, (k1 - 1) & ~7) / p.BS];
+  };
+  constexpr bool PF = BF && VP <= 128;   // (wider values fill the registers: their K rows are requested map by map when needed)
+  uint4_t kf[PF ? 2 : 1][2][KS];
+  auto load_k = [&](int kb, int m0, int m1) {
 #pragma unroll
     for (int t = 0; t < 2; ++t) {
       const int key = min(kb + krow + 4 * t, k1 - 1);
-      kr[t] = kc + (((long)bt[key / p.BS] * p.G + kvh) * p.BS + key % p.BS) * 2 * p.dim;
-    }
-    const int vk = kb + 8 * g < k1 ? kb + 8 * g : ((k1 - 1) & ~7);
-    const T* vrow = vc + ((long)bt[vk / p.BS] * p.G + kvh) * p.vdim * p.BS + vk % p.BS;
-    uint4_t vf[BF ? VT : 1];
-    floatx4 c[2][2];
+      const T* kr = kc + (((long)pk[t] * p.G + kvh) * p.BS + key % p.BS) * 2 * p.dim;
 #pragma unroll
-    for (int mp = 0; mp < 2; ++mp) {
-      uint4_t kf[2][KS];
-#pragma unroll
-      for (int t = 0; t < 2; ++t)
+      for (int mp = m0; mp < m1; ++mp)
 #pragma unroll
         for (int s = 0; s < KS; ++s) {
           const int d0 = s * 4 * EV + g * EV;
-          kf[t][s] = d0 < p.dim ? ld16(kr[t] + mp * p.dim + d0) : uint4_t{0u, 0u, 0u, 0u};
+          kf[PF ? mp : 0][t][s] = d0 < p.dim ? ld16(kr + mp * p.dim + d0) : uint4_t{0u, 0u, 0u, 0u};
         }
-      if constexpr (BF) {
-        if (mp == 0) {
+    }
+  };
+  int kb = k0 + 32 * step0;
+  if (kb >= k1) return;
+  pages(kb);
+  if (PF) load_k(kb, 0, 2);
+  for (; kb < k1; kb += 32 * stride) {
+    const int vk = min(kb + 8 * g, (k1 - 1) & ~7), kn = kb + 32 * stride;
+    const T* vrow = vc + ((long)pv * p.G + kvh) * p.vdim * p.BS + vk % p.BS;
+    uint4_t vf[BF ? VT : 1];
+    if constexpr (BF) {
 #pragma unroll
-          for (int vt = 0; vt < VT; ++vt) {
-            const int vd = vt * 16 + n16;
-            vf[vt] = vd < p.vdim ? ld16(vrow + (long)vd * p.BS) : uint4_t{0u, 0u, 0u, 0u};
-          }
-        }
+      for (int vt = 0; vt < VT; ++vt) {
+        const int vd = vt * 16 + n16;
+        vf[vt] = vd < p.vdim ? ld16(vrow + (long)vd * p.BS) : uint4_t{0u, 0u, 0u, 0u};
       }
+    }
+    if (PF && kn < k1) pages(kn);
+    floatx4 c[2][2];
+#pragma unroll
+    for (int mp = 0; mp < 2; ++mp) {
+      if (!PF) load_k(kb, mp, mp + 1);
 #pragma unroll
       for (int t = 0; t < 2; ++t) {
         c[mp][t] = floatx4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int s = 0; s < KS; ++s) c[mp][t] = mma_qk<T>(kf[t][s], qf[mp][s], c[mp][t]);
+        for (int s = 0; s < KS; ++s) c[mp][t] = mma_qk<T>(kf[PF ? mp : 0][t][s], qf[mp][s], c[mp][t]);
       }
+    }
+    if (kn < k1) {
+      if (PF) load_k(kn, 0, 2);
+      else pages(kn);
     }
     short8 pbits[2];
     float pw[2][2][4];
@@ -270,7 +288,7 @@ __global__ __launch_bounds__(256) void diff_prefill_kernel(DiffParams p, const i
 // ---- decode: workgroup = (sequence, up to 16 heads of one kv group, key split z)
 // part: [B, H, Z, 2, vdim + 2] f32 = O^T of a map relative to m, then m, l
 template <typename T, int KP, int VP>
-__global__ __launch_bounds__(256) void diff_decode_kernel(DiffParams p, const int* __restrict__ ctx_lens, int Z, T* __restrict__ out, long os,
+__global__ __launch_bounds__(256, sizeof(T) == 2 && VP <= 128 && KP <= 64 ? 2 : 1) void diff_decode_kernel(DiffParams p, const int* __restrict__ ctx_lens, int Z, T* __restrict__ out, long os,
                                                           float* __restrict__ part) {
   constexpr int VT = VP / 16;
   constexpr bool EXACT = sizeof(T) == 4;

@@ -376,6 +376,54 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
   }
 }
 
+// The same with 16-byte (f32) / 8-byte (bf16) accesses: LPH adjacent lanes hold a head, 4 columns each (dv = 4 LPH at most, dv % 4 == 0)
+template <typename TG, typename TO, int LPH>
+__global__ __launch_bounds__(256) void head_norm_gate_vec_kernel(const float* __restrict__ o, long os, const TG* __restrict__ g, long gs,
+                                                                 const float* __restrict__ w, int H, int dv, float eps, int kind,
+                                                                 TO* __restrict__ out, long outs) {
+  const long t = blockIdx.x;
+  const int c = 4 * (threadIdx.x % LPH);
+  auto ld4 = [](const auto* p, float (&f)[4]) {
+    using E = std::remove_cv_t<std::remove_reference_t<decltype(*p)>>;
+    if constexpr (sizeof(E) == 4) {
+      const floatx4 v = *reinterpret_cast<const floatx4*>(p);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) f[e] = v[e];
+    } else {
+      const short4_t v = *reinterpret_cast<const short4_t*>(p);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) f[e] = bf2f((bf16_t)v[e]);
+    }
+  };
+  for (int h = threadIdx.x / LPH; h < (H + 256 / LPH - 1) / (256 / LPH) * (256 / LPH); h += 256 / LPH) {   // (whole waves stay together)
+    const bool in = h < H && c < dv;
+    const long hc = (long)min(h, H - 1) * dv + min(c, dv - 4);
+    float x[4], gv[4], ww[4] = {1.f, 1.f, 1.f, 1.f};
+    ld4(o + t * os + hc, x);
+    ld4(g + t * gs + hc, gv);
+    if (w) ld4(w + hc, ww);
+    float ss = in ? (x[0] * x[0] + x[1] * x[1]) + (x[2] * x[2] + x[3] * x[3]) : 0.f;
+#pragma unroll
+    for (int d = LPH / 2; d > 0; d >>= 1) ss += __shfl_xor(ss, d, 64);
+    const float inv = 1.f / sqrtf(ss / (float)dv + eps);
+    if (!in) continue;
+    float r[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const float s = sigmoid_f(gv[e]);
+      r[e] = x[e] * inv * ww[e] * (kind == 0 ? gv[e] * s : s);
+    }
+    if constexpr (sizeof(TO) == 4) {
+      *reinterpret_cast<floatx4*>(out + t * outs + hc) = floatx4{r[0], r[1], r[2], r[3]};
+    } else {
+      short4_t v;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = (short)f2bf(r[e]);
+      *reinterpret_cast<short4_t*>(out + t * outs + hc) = v;
+    }
+  }
+}
+
 // The same for fewer heads than waves (one norm over a long row): the whole workgroup takes each head in turn
 template <typename TG, typename TO>
 __global__ __launch_bounds__(256) void row_norm_gate_kernel(const float* __restrict__ o, long os, const TG* __restrict__ g, long gs,
@@ -455,8 +503,16 @@ int lk_head_norm_gate(const float* o, long os, const void* g, long gs, int g_esz
                       int kind, void* out, long outs, int out_esz, hipStream_t st) {
   if (T <= 0) return 0;
   if (kind != 0 && kind != 1) return -1;
+  const auto al = [](const void* x, int b) { return reinterpret_cast<uintptr_t>(x) % b == 0; };
+  const bool vec = dv % 4 == 0 && dv <= 256 && os % 4 == 0 && gs % 4 == 0 && outs % 4 == 0 && al(o, 16) && al(w, 16) && al(g, 4 * g_esz) && al(out, 4 * out_esz);
 #define LK_HNG(TG, TO)                                                                                                          \
-  if (H < 4 && dv >= 256)                                                                                                       \
+  if (H >= 4 && vec && dv > 128)                                                                                                \
+    head_norm_gate_vec_kernel<TG, TO, 64><<<(unsigned)T, 256, 0, st>>>(o, os, (const TG*)g, gs, w, H, dv, eps, kind, (TO*)out, outs); \
+  else if (H >= 4 && vec && dv > 64)                                                                                            \
+    head_norm_gate_vec_kernel<TG, TO, 32><<<(unsigned)T, 256, 0, st>>>(o, os, (const TG*)g, gs, w, H, dv, eps, kind, (TO*)out, outs); \
+  else if (H >= 4 && vec && dv > 32)                                                                                            \
+    head_norm_gate_vec_kernel<TG, TO, 16><<<(unsigned)T, 256, 0, st>>>(o, os, (const TG*)g, gs, w, H, dv, eps, kind, (TO*)out, outs); \
+  else if (H < 4 && dv >= 256)                                                                                                  \
     row_norm_gate_kernel<TG, TO><<<(unsigned)T, 256, 0, st>>>(o, os, (const TG*)g, gs, w, H, dv, eps, kind, (TO*)out, outs);   \
   else                                                                                                                          \
     head_norm_gate_kernel<TG, TO><<<(unsigned)T, 256, 0, st>>>(o, os, (const TG*)g, gs, w, H, dv, eps, kind, (TO*)out, outs)

@@ -57,7 +57,7 @@ struct HeadDeltaParams {
 // ---- single tokens.  512 (256) threads = 32 (16) groups of 4 adjacent state columns x 16 row slices; a thread holds the rows rs,
 // rs + 16, ... of its 4 columns (16-byte accesses, VEC), and the workgroup walks the head's columns in blocks of 128 (64).
 template <typename T, int NR, int CGN, bool VEC>
-__global__ __launch_bounds__(16 * CGN) void head_delta_step_kernel(HeadDeltaParams p) {
+__global__ __launch_bounds__(16 * CGN, NR <= 8 ? 4 : 2) void head_delta_step_kernel(HeadDeltaParams p) {
   constexpr int NT = 16 * CGN, NW = NT / 64, COLS = 4 * CGN;
   __shared__ float sq[NR * 16], sk[NR * 16], red[NW][CGN][9], so[1024];
   const int s = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
@@ -464,6 +464,251 @@ __global__ __launch_bounds__(64 * NW) void head_delta_chunk_kernel(HeadDeltaPara
   }
 }
 
+// The same chain for bf16 rows.  A bf16 row times the f32 state is exact as three bf16 products: the state is split into parts of 8
+// mantissa bits (s = hi + mid + lo, each cut off, so the sum is s itself), and the MFMA sums the exact partial products in f32.  One
+// 32-row step of the products with the state is then 3 MFMAs of 16 cycles instead of 8 of 32.
+//
+// LDS rows of q and k hold, per 32 channels, the order of the B operand that the state's accumulators give without a move: place 8 g + e
+// is channel 4 g + e (e < 4) and 16 + 4 g + e - 4 (e >= 4).  The same rows read transposed (4 tokens x 16 channels at a time) feed
+// the update; its B operand holds u's parts hi and mid of the same 4 tokens side by side, then lo beside zeros.
+typedef short4_t __attribute__((address_space(3))) * lds_short4_ptr;
+
+LK_DEVICE unsigned upper_halves(float a, float b) {   // bf16 cut-offs of a (low half) and b (high half)
+  return __builtin_amdgcn_perm(__float_as_uint(b), __float_as_uint(a), 0x07060302u);
+}
+LK_DEVICE float cut(float v) { return __uint_as_float(__float_as_uint(v) & 0xffff0000u); }
+
+template <int NR, int NW, bool VEC>
+__global__ __launch_bounds__(64 * NW) void head_delta_chunk_bf16_kernel(HeadDeltaParams p) {
+  static_assert(NR % 2 == 0, "32-row steps");
+  constexpr int NP = NR * 16, NB = NR / 2, LH = NP + 24, NT = 64 * NW, COLS = 16 * NW;
+  __shared__ __attribute__((aligned(16))) bf16_t hk[2][kL][LH];
+  __shared__ __attribute__((aligned(16))) bf16_t hq[2][kL][LH];
+  __shared__ __attribute__((aligned(16))) float sv[2][kL][COLS + 4];
+  __shared__ __attribute__((aligned(16))) float sp[2][kL][kPre];
+  const int s = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, j0 = blockIdx.z * COLS;
+  const int lane = tid & 63, w = tid >> 6, n16 = lane & 15, g = lane >> 4;
+  const int col = j0 + 16 * w + n16;
+  const bool cv = col < p.dv;
+  const int row0 = p.cu[s], len = p.cu[s + 1] - row0, slot = p.slots[s];
+  if (len <= 0) return;
+  float* og = p.o + (long)row0 * p.H * p.dv + (long)h * p.dv;
+  if (slot < 0) {
+    for (int i = tid; i < len * COLS; i += NT) {
+      const int c = j0 + i % COLS;
+      if (c < p.dv) og[(long)(i / COLS) * p.H * p.dv + c] = 0.f;
+    }
+    return;
+  }
+  const bool fresh = p.positions[row0] == 0;
+  float* Sg = p.state + ((long)slot * p.H + h) * p.dk * p.dv + (cv ? col : 0);
+  floatx4 S[NR];
+#pragma unroll
+  for (int nt = 0; nt < NR; ++nt) S[nt] = floatx4{0.f, 0.f, 0.f, 0.f};
+  if (!fresh) {   // (loads from clamped places, selected afterwards: all in flight together)
+#pragma unroll
+    for (int nt = 0; nt < NR; ++nt)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) S[nt][j] = Sg[(long)min(nt * 16 + 4 * g + j, p.dk - 1) * p.dv];
+#pragma unroll
+    for (int nt = 0; nt < NR; ++nt)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) S[nt][j] = cv && nt * 16 + 4 * g + j < p.dk ? S[nt][j] : 0.f;
+  }
+  const int kh = h / (p.H / p.Hk);
+  const bf16_t* qg = reinterpret_cast<const bf16_t*>(p.q) + (long)kh * p.dk;
+  const bf16_t* kg = reinterpret_cast<const bf16_t*>(p.k) + (long)kh * p.dk;
+  const bf16_t* vg = reinterpret_cast<const bf16_t*>(p.v) + (long)h * p.dv;
+  const float* pg = p.pre + ((long)row0 * p.H + h) * kPre;
+  // A chunk's operands travel into registers two chunks ahead, as raw pieces from clamped places, and are masked as they are staged.
+  constexpr int CPR = NP / 8, NQK = (2 * kL * CPR + NT - 1) / NT, NV = (kL * COLS / 4 + NT - 1) / NT, NPR = (kL * kPre / 4 + NT - 1) / NT;
+  struct Raw {
+    uint4_t qk[NQK];
+    bf16_t v[NV][4];
+    floatx4 pre[NPR];
+  };
+  auto fetch = [&](int t0, Raw& r) __attribute__((always_inline)) {
+    if (t0 >= len) return;
+    const int tl = min(kL, len - t0), ncpr = p.dk / 8;
+    if constexpr (VEC) {
+#pragma unroll
+      for (int x = 0; x < NQK; ++x) {
+        const int i = min(tid + NT * x, 2 * kL * CPR - 1), which = i / (kL * CPR), e = i % (kL * CPR);
+        const int t = min(e / CPR, tl - 1), c = min(e % CPR, ncpr - 1);
+        r.qk[x] = ld16((which ? qg : kg) + (long)(row0 + t0 + t) * (which ? p.qs : p.ks) + c * 8);
+      }
+    }
+#pragma unroll
+    for (int x = 0; x < NV; ++x) {
+      const int i = min(tid + NT * x, kL * COLS / 4 - 1), t = min(i / (COLS / 4), tl - 1), c = j0 + 4 * (i % (COLS / 4));
+      const bf16_t* vr = vg + (long)(row0 + t0 + t) * p.vs;
+      if constexpr (VEC) {
+        *reinterpret_cast<short4_t*>(r.v[x]) = *reinterpret_cast<const short4_t*>(vr + min(c, p.dv - 4));
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) r.v[x][e] = vr[min(c + e, p.dv - 1)];
+      }
+    }
+#pragma unroll
+    for (int x = 0; x < NPR; ++x) {
+      const int i = min(tid + NT * x, kL * kPre / 4 - 1), t = min(i / (kPre / 4), tl - 1), c = i % (kPre / 4);
+      r.pre[x] = *reinterpret_cast<const floatx4*>(pg + (long)(t0 + t) * p.H * kPre + 4 * c);
+    }
+  };
+  auto stage = [&](int t0, int buf, const Raw& r) __attribute__((always_inline)) {
+    if (t0 >= len) return;
+    const int tl = min(kL, len - t0);
+    if constexpr (VEC) {
+#pragma unroll
+      for (int x = 0; x < NQK; ++x) {
+        const int i = tid + NT * x;
+        if (2 * kL * CPR % NT == 0 || i < 2 * kL * CPR) {
+          const int which = i / (kL * CPR), e = i % (kL * CPR), t = e / CPR, c = e % CPR;
+          bf16_t* dst = (which ? hq[buf][t] : hk[buf][t]) + 32 * (c >> 2) + 16 * (c & 1) + 4 * ((c >> 1) & 1);
+          const uint4_t raw = t >= tl || c >= p.dk / 8 ? uint4_t{0u, 0u, 0u, 0u} : r.qk[x];
+          *reinterpret_cast<uint64_t*>(dst) = (uint64_t)raw[1] << 32 | raw[0];
+          *reinterpret_cast<uint64_t*>(dst + 8) = (uint64_t)raw[3] << 32 | raw[2];
+        }
+      }
+    } else {
+      for (int i = tid; i < 2 * kL * NP; i += NT) {
+        const int which = i / (kL * NP), e = i % (kL * NP), t = e / NP, c = e % NP;
+        const long row = row0 + t0 + t;
+        bf16_t v = 0;
+        if (t < tl && c < p.dk) v = which ? qg[row * p.qs + c] : kg[row * p.ks + c];
+        (which ? hq[buf][t] : hk[buf][t])[(c & ~31) + 8 * ((c >> 2) & 3) + 4 * ((c >> 4) & 1) + (c & 3)] = v;
+      }
+    }
+#pragma unroll
+    for (int x = 0; x < NV; ++x) {
+      const int i = tid + NT * x;
+      if (kL * COLS / 4 % NT == 0 || i < kL * COLS / 4) {
+        const int t = i / (COLS / 4), c = 4 * (i % (COLS / 4));
+        floatx4 v;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = t < tl && j0 + c + e < p.dv ? bf2f(r.v[x][e]) : 0.f;
+        *reinterpret_cast<floatx4*>(&sv[buf][t][c]) = v;
+      }
+    }
+#pragma unroll
+    for (int x = 0; x < NPR; ++x) {
+      const int i = tid + NT * x;
+      if (kL * kPre / 4 % NT == 0 || i < kL * kPre / 4) {
+        const int t = i / (kPre / 4), c = i % (kPre / 4);
+        *reinterpret_cast<floatx4*>(&sp[buf][t][4 * c]) = t < tl ? r.pre[x] : floatx4{0.f, 0.f, 0.f, 0.f};
+      }
+    }
+  };
+  uint4_t part[NB][3];   // the state's parts as B operands
+  auto split = [&]() __attribute__((always_inline)) {
+#pragma unroll
+    for (int b = 0; b < NB; ++b)
+#pragma unroll
+      for (int x = 0; x < 4; ++x) {
+        float a = S[2 * b + (x >> 1)][2 * (x & 1)], c = S[2 * b + (x >> 1)][2 * (x & 1) + 1];
+        part[b][0][x] = upper_halves(a, c);
+        a -= cut(a);
+        c -= cut(c);
+        part[b][1][x] = upper_halves(a, c);
+        a -= cut(a);
+        c -= cut(c);
+        part[b][2][x] = upper_halves(a, c);
+      }
+  };
+  auto mma = [](uint4_t a, uint4_t b, floatx4 c) __attribute__((always_inline)) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(short8, a), __builtin_bit_cast(short8, b), c, 0, 0, 0);
+  };
+  const int qq = n16 >> 2, pp = n16 & 3;
+  auto compute = [&](int t0, int buf) __attribute__((always_inline)) {
+    const int tl = min(kL, len - t0);
+    // K S and Q S: rows t = 4g + j, column n16 of this wave's tile
+    floatx4 y1[3], y2[3];
+#pragma unroll
+    for (int x = 0; x < 3; ++x) y1[x] = y2[x] = floatx4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+      const uint4_t kf = ld16(&hk[buf][n16][32 * b + 8 * g]);
+#pragma unroll
+      for (int x = 0; x < 3; ++x) y1[x] = mma(kf, part[b][x], y1[x]);
+    }
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+      const uint4_t qf = ld16(&hq[buf][n16][32 * b + 8 * g]);
+#pragma unroll
+      for (int x = 0; x < 3; ++x) y2[x] = mma(qf, part[b][x], y2[x]);
+    }
+    float xv[4];
+    floatx4 f4[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      f4[j] = *reinterpret_cast<const floatx4*>(&sp[buf][4 * g + j][32]);
+      xv[j] = sv[buf][4 * g + j][16 * w + n16] - f4[j][0] * (y1[0][j] + (y1[1][j] + y1[2][j]));
+    }
+    floatx4 u = {0.f, 0.f, 0.f, 0.f}, o;
+    const floatx4 b4 = *reinterpret_cast<const floatx4*>(&sp[buf][n16][4 * g]), p4 = *reinterpret_cast<const floatx4*>(&sp[buf][n16][16 + 4 * g]);
+    const float dec = sp[buf][0][35];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) u = __builtin_amdgcn_mfma_f32_16x16x4f32(b4[j], xv[j], u, 0, 0, 0);
+#pragma unroll
+    for (int nt = 0; nt < NR; ++nt)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) S[nt][j] *= dec;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o[j] = f4[j][1] * (y2[0][j] + (y2[1][j] + y2[2][j]));
+    // state: rows i = 16 nt + 4g + j, column n16
+    float us[4], r1[4], r2[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      us[j] = u[j] * f4[j][2];
+      r1[j] = us[j] - cut(us[j]);
+      r2[j] = r1[j] - cut(r1[j]);
+    }
+    const uint4_t ub = {upper_halves(us[0], us[1]), upper_halves(us[2], us[3]), upper_halves(r1[0], r1[1]), upper_halves(r1[2], r1[3])};
+    const uint4_t ul = {upper_halves(r2[0], r2[1]), upper_halves(r2[2], r2[3]), 0u, 0u};
+#pragma unroll
+    for (int nt = 0; nt < NR; ++nt) {
+      const bf16_t* a0 = &hk[buf][4 * g + qq][32 * (nt >> 1) + 8 * pp + 4 * (nt & 1)];
+      const uint64_t kt = __builtin_bit_cast(uint64_t, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4_ptr)(a0)));
+      const uint4_t ka = {(unsigned)kt, (unsigned)(kt >> 32), (unsigned)kt, (unsigned)(kt >> 32)};
+      S[nt] = mma(ka, ub, S[nt]);
+      S[nt] = mma(ka, ul, S[nt]);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o = __builtin_amdgcn_mfma_f32_16x16x4f32(p4[j], u[j], o, 0, 0, 0);
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (cv && 4 * g + j < tl) og[(long)(t0 + 4 * g + j) * p.H * p.dv + col] = o[j];
+    split();
+  };
+  Raw ra, rb;
+  fetch(0, ra);
+  fetch(kL, rb);
+  split();
+  stage(0, 0, ra);
+  fetch(2 * kL, ra);
+  __syncthreads();
+  for (int t0 = 0; t0 < len; t0 += 2 * kL) {
+    compute(t0, 0);
+    stage(t0 + kL, 1, rb);
+    fetch(t0 + 3 * kL, rb);
+    __syncthreads();
+    if (t0 + kL >= len) break;
+    compute(t0 + kL, 1);
+    stage(t0 + 2 * kL, 0, ra);
+    fetch(t0 + 4 * kL, ra);
+    __syncthreads();
+  }
+  if (cv) {
+#pragma unroll
+    for (int nt = 0; nt < NR; ++nt)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int i = nt * 16 + 4 * g + j;
+        if (i < p.dk) Sg[(long)i * p.dv] = S[nt][j];
+      }
+  }
+}
+
 bool al(const void* x, int b) { return reinterpret_cast<uintptr_t>(x) % b == 0; }
 
 template <typename T, int NR>
@@ -484,8 +729,14 @@ int launch_step(const HeadDeltaParams& p, int S, hipStream_t st) {
 template <typename T, int NR, int NW>
 int launch_chunk(const HeadDeltaParams& p, int S, bool vec, hipStream_t st) {
   const dim3 grid((unsigned)S, (unsigned)p.H, (unsigned)((p.dv + 16 * NW - 1) / (16 * NW)));
-  if (vec) head_delta_chunk_kernel<T, NR, NW, true><<<grid, 64 * NW, 0, st>>>(p);
-  else head_delta_chunk_kernel<T, NR, NW, false><<<grid, 64 * NW, 0, st>>>(p);
+  if constexpr (sizeof(T) == 2) {
+    constexpr int N2 = NR < 2 ? 2 : NR;
+    if (vec) head_delta_chunk_bf16_kernel<N2, NW, true><<<grid, 64 * NW, 0, st>>>(p);
+    else head_delta_chunk_bf16_kernel<N2, NW, false><<<grid, 64 * NW, 0, st>>>(p);
+  } else {
+    if (vec) head_delta_chunk_kernel<T, NR, NW, true><<<grid, 64 * NW, 0, st>>>(p);
+    else head_delta_chunk_kernel<T, NR, NW, false><<<grid, 64 * NW, 0, st>>>(p);
+  }
   LK_CHECK_LAUNCH();
   return 0;
 }

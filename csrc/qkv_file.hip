@@ -5,7 +5,8 @@
 // [blocks, G, BS, dim], v to the key-contiguous one [blocks, G, vdim, BS], at slots[t] (< 0: nothing is cached).
 //
 // One workgroup per token.  A thread holds 16-byte pieces of the row (a pair never straddles two pieces: heads are multiples of a
-// piece), so the row is read once and everything between load and store is in registers.
+// piece), so the row is read once and everything between load and store is in registers.  With many rows the values are filed by a kernel
+// of their own: 16 tokens x 64 columns turn round in LDS, so that a column's run of tokens is written in 16-byte pieces.
 #include "common.h"
 #include "kernels.h"
 #include "attn_frag.h"
@@ -29,6 +30,7 @@ struct FileParams {
   void* kc;
   void* vc;
   const int* slots;
+  int v_apart;         // the values are filed by file_values_kernel
 };
 
 template <typename T, int MAXC>
@@ -37,7 +39,7 @@ __global__ __launch_bounds__(256) void qkv_file_kernel(FileParams p) {
   __shared__ float scs[kMaxRot / 2], ssn[kMaxRot / 2], red[4];
   const long t = blockIdx.x;
   const int tid = threadIdx.x, slot = p.slots[t];
-  const int nq = p.H * p.dim, nk = p.G * p.dim, n = nq + nk + p.G * p.vdim;
+  const int nq = p.H * p.dim, nk = p.G * p.dim, n = nq + nk + (p.v_apart ? 0 : p.G * p.vdim);
   T* row = reinterpret_cast<T*>(p.u) + t * p.us;
   for (int i = tid; i < p.rot / 2; i += 256) {
     float sn, cs;
@@ -118,9 +120,54 @@ __global__ __launch_bounds__(256) void qkv_file_kernel(FileParams p) {
   }
 }
 
+// grid (16 tokens, 64 value columns), 128 threads
+constexpr int kVTok = 16, kVCol = 64;
 template <typename T>
-int launch_file(const FileParams& p, long T_, hipStream_t st) {
-  const int n = (p.H + p.G) * p.dim + p.G * p.vdim, per = 256 * El<T>::V;
+__global__ __launch_bounds__(128) void file_values_kernel(FileParams p, long rows) {
+  constexpr int EV = El<T>::V;
+  __shared__ __attribute__((aligned(16))) T sv[kVCol][kVTok + EV];
+  const int tid = threadIdx.x, nv = p.G * p.vdim, c0 = blockIdx.y * kVCol, v0 = (p.H + p.G) * p.dim;
+  const long t0 = (long)blockIdx.x * kVTok;
+  const int tl = (int)min((long)kVTok, rows - t0);
+  for (int i = tid; i < kVTok * kVCol / EV; i += 128) {
+    const int t = i / (kVCol / EV), c = (i % (kVCol / EV)) * EV;
+    if (t < tl && c0 + c < nv) {   // (nv is a multiple of a piece)
+      const uint4_t raw = ld16(reinterpret_cast<const T*>(p.u) + (t0 + t) * p.us + v0 + c0 + c);
+      const T* e = reinterpret_cast<const T*>(&raw);
+#pragma unroll
+      for (int j = 0; j < EV; ++j) {
+        if (p.bias) El<T>::st(&sv[c + j][t], El<T>::ld(e + j) + p.bias[v0 + c0 + c + j]);
+        else sv[c + j][t] = e[j];
+      }
+    }
+  }
+  __syncthreads();
+  for (int i = tid; i < kVCol * kVTok / EV; i += 128) {
+    const int c = i / (kVTok / EV), tb = (i % (kVTok / EV)) * EV;
+    if (c0 + c >= nv || tb >= tl) continue;
+    const int gh = (c0 + c) / p.vdim, d = (c0 + c) % p.vdim, n = min(EV, tl - tb), s0 = p.slots[t0 + tb];
+    auto place = [&](int slot) { return reinterpret_cast<T*>(p.vc) + (((long)(slot / p.BS) * p.G + gh) * p.vdim + d) * p.BS + slot % p.BS; };
+    bool run = n == EV && s0 >= 0 && s0 % EV == 0;
+    for (int j = 1; j < n; ++j) run = run && p.slots[t0 + tb + j] == s0 + j;
+    if (run) {
+      *reinterpret_cast<uint4_t*>(place(s0)) = *reinterpret_cast<const uint4_t*>(&sv[c][tb]);
+    } else {
+      for (int j = 0; j < n; ++j) {
+        const int slot = p.slots[t0 + tb + j];
+        if (slot >= 0) *place(slot) = sv[c][tb + j];
+      }
+    }
+  }
+}
+
+template <typename T>
+int launch_file(FileParams p, long T_, hipStream_t st) {
+  p.v_apart = T_ >= 256 && p.BS % El<T>::V == 0 && (reinterpret_cast<uintptr_t>(p.vc) & 15) == 0;
+  if (p.v_apart) {
+    file_values_kernel<T><<<dim3((unsigned)((T_ + kVTok - 1) / kVTok), (unsigned)((p.G * p.vdim + kVCol - 1) / kVCol)), 128, 0, st>>>(p, T_);
+    LK_CHECK_LAUNCH();
+  }
+  const int n = (p.H + p.G) * p.dim + (p.v_apart ? 0 : p.G * p.vdim), per = 256 * El<T>::V;
   const unsigned g = (unsigned)T_;
   if (n <= per) qkv_file_kernel<T, 1><<<g, 256, 0, st>>>(p);
   else if (n <= 2 * per) qkv_file_kernel<T, 2><<<g, 256, 0, st>>>(p);
@@ -146,6 +193,6 @@ int lk_qkv_file(void* u, long us, long T, int H, int G, int dim, int vdim, const
   FileParams p;
   p.u = u; p.us = us; p.H = H; p.G = G; p.dim = dim; p.vdim = vdim; p.BS = BS; p.bias = bias; p.qw = qw; p.kw = kw;
   p.inv_nq = qw ? 1.f / (float)norm_q : 0.f; p.inv_nk = qw ? 1.f / (float)norm_k : 0.f;
-  p.eps = eps; p.rot = rot; p.freq = freq; p.mag = mag; p.positions = positions; p.kc = kc; p.vc = vc; p.slots = slots;
+  p.eps = eps; p.rot = rot; p.freq = freq; p.mag = mag; p.positions = positions; p.kc = kc; p.vc = vc; p.slots = slots; p.v_apart = 0;
   return esz == 2 ? launch_file<bf16_t>(p, T, st) : launch_file<float>(p, T, st);
 }

@@ -120,11 +120,18 @@ __global__ __launch_bounds__(256) void conv_silu_vec_kernel(const T* __restrict_
   }
   const bool past = positions[row0] > 0;
   float wk[4][EV], b[EV], win[3][EV];
+  const bool w4 = taps == 4 && (reinterpret_cast<uintptr_t>(w) & 15) == 0;   // a channel's taps in one 16-byte load
 #pragma unroll
   for (int e = 0; e < EV; ++e) {
     b[e] = bias ? bias[c0 + e] : 0.f;
+    if (w4) {
+      const floatx4 v = *reinterpret_cast<const floatx4*>(w + (long)(c0 + e) * 4);
 #pragma unroll
-    for (int k = 0; k < 4; ++k) wk[k][e] = k >= 4 - taps ? w[(long)(c0 + e) * taps + (k - (4 - taps))] : 0.f;
+      for (int k = 0; k < 4; ++k) wk[k][e] = v[k];
+    } else {
+#pragma unroll
+      for (int k = 0; k < 4; ++k) wk[k][e] = k >= 4 - taps ? w[(long)(c0 + e) * taps + (k - (4 - taps))] : 0.f;
+    }
   }
 #pragma unroll
   for (int d = 3; d >= 1; --d) {  // win[3 - d] = the input d tokens before the tile's first
@@ -136,18 +143,25 @@ __global__ __launch_bounds__(256) void conv_silu_vec_kernel(const T* __restrict_
       else if (past && si >= 0) ldrow(state + ((long)slot * (taps - 1) + si) * C + c0, win[3 - d]);
     }
   }
-  for (int i = i0; i < i1; ++i) {
-    float cur[EV], r[EV];
-    ldrow(u + (long)(row0 + i) * us + c0, cur);
+  // (rows in groups of four, requested together: the window slides over values in registers)
+  for (int i = i0; i < i1; i += 4) {
+    float cur[4][EV];
 #pragma unroll
-    for (int e = 0; e < EV; ++e) {
-      const float acc = b[e] + wk[0][e] * win[0][e] + wk[1][e] * win[1][e] + wk[2][e] * win[2][e] + wk[3][e] * cur[e];
-      r[e] = act ? silu_f<sizeof(T) == 4>(acc) : acc;
-      win[0][e] = win[1][e];
-      win[1][e] = win[2][e];
-      win[2][e] = cur[e];
+    for (int x = 0; x < 4; ++x) ldrow(u + (long)(row0 + min(i + x, i1 - 1)) * us + c0, cur[x]);
+#pragma unroll
+    for (int x = 0; x < 4; ++x) {
+      if (i + x >= i1) break;
+      float r[EV];
+#pragma unroll
+      for (int e = 0; e < EV; ++e) {
+        const float acc = b[e] + wk[0][e] * win[0][e] + wk[1][e] * win[1][e] + wk[2][e] * win[2][e] + wk[3][e] * cur[x][e];
+        r[e] = act ? silu_f<sizeof(T) == 4>(acc) : acc;
+        win[0][e] = win[1][e];
+        win[1][e] = win[2][e];
+        win[2][e] = cur[x][e];
+      }
+      strow(out + (long)(row0 + i + x) * os + c0, r);
     }
-    strow(out + (long)(row0 + i) * os + c0, r);
   }
 }
 

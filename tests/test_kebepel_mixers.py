@@ -310,15 +310,26 @@ def test_attention_kernels_of_all_instances(shape, climb, device, dtype):
 @pytest.mark.parametrize("H,G,dim,vdim,rot,page", [(4, 2, 48, 32, 48, 16), (3, 1, 24, 40, 16, 48), (16, 4, 128, 128, 64, 16), (6, 6, 16, 8, 0, 32)])
 def test_queries_keys_values_filed(H, G, dim, vdim, rot, page, device, dtype):
     """Bias, norm over the whole projection (one loud head sets the root of all), pair rotation at positions up to 3,000 and the paged
-    write at scattered slots, with and without norm; a padding row's slot files nothing."""
+    write at scattered slots, with and without norm; a padding row's slot files nothing.  Few rows, and many (whose values take
+    their own way): runs of slots that start on and off 16-byte borders, cut by pages, and single scattered ones."""
     g = torch.Generator().manual_seed(H)
-    T, n = 21, (H + G) * dim + G * vdim
+    for T in (21, 300):
+        filed(H, G, dim, vdim, rot, page, device, dtype, g, T)
+
+
+def filed(H, G, dim, vdim, rot, page, device, dtype, g, T):
+    n, NB = (H + G) * dim + G * vdim, 500 // page
     u = q16(rnd(g, T, n))
     u[:, :dim] *= 8                                          # a norm per head would not see it in the others
     bias, qw, kw = (rnd(g, s).float().double() for s in (n, H * dim, G * dim))
     freq = (torch.rand(max(rot // 2, 1), generator=g, dtype=torch.float64) * 0.5).float().double()
     pos = torch.randint(0, 3000, (T,), generator=g, dtype=torch.int32)
-    slots = torch.randperm(4 * page, generator=g)[:T].int()
+    slots = torch.randperm(NB * page, generator=g)[:T].int()
+    if T > 100:     # tokens in order in pages out of order, from an odd offset on, some scattered
+        order = torch.randperm(NB, generator=g)
+        lin = (order.view(-1, 1) * page + torch.arange(page)).reshape(-1).int()
+        slots[:200], slots[200:] = lin[:200], lin[205:205 + T - 200]
+        slots[17:23] = lin[400:406].flip(0)
     slots[4] = -1
     for norm in (True, False):
         x = u + bias
@@ -333,13 +344,13 @@ def test_queries_keys_values_filed(H, G, dim, vdim, rot, page, device, dtype):
                 t[..., 0:rot:2], t[..., 1:rot:2] = 1.2 * (a * ang.cos() - b * ang.sin()), 1.2 * (b * ang.cos() + a * ang.sin())
         ud = torch.zeros(T, n + 8, dtype=dtype, device=device)
         ud[:, 8:] = u.to(dtype).to(device)
-        kc, vc = torch.zeros(4, G, page, dim, dtype=dtype, device=device), torch.zeros(4, G, vdim, page, dtype=dtype, device=device)
+        kc, vc = torch.zeros(NB, G, page, dim, dtype=dtype, device=device), torch.zeros(NB, G, vdim, page, dtype=dtype, device=device)
         f = lambda t: t.float().to(device)      # noqa: E731
         ops.qkv_file(ud, 8, H, G, dim, vdim, f(bias), f(qw) if norm else None, f(kw) if norm else None, H * dim - 3, G * dim - 1, EPS, rot, f(freq), 1.2,
                      pos.to(device), kc, vc, slots.to(device))
         bound = 2e-5 if dtype == torch.float32 else 8e-3
         assert rel_err(ud[:, 8:8 + H * dim], q.reshape(T, -1)) < bound
-        wk, wv = torch.zeros(4, G, page, dim, dtype=torch.float64), torch.zeros(4, G, vdim, page, dtype=torch.float64)
+        wk, wv = torch.zeros(NB, G, page, dim, dtype=torch.float64), torch.zeros(NB, G, vdim, page, dtype=torch.float64)
         for t in range(T):
             if int(slots[t]) >= 0:
                 wk[slots[t] // page, :, slots[t] % page], wv[slots[t] // page, :, :, slots[t] % page] = k[t], v[t]
@@ -464,7 +475,12 @@ def test_sandwiched_layer_norms(W, device, dtype):
     """Norm of the result, sum, step vector and next norm in one pass, each part present or absent; rows chosen by an index leave the
     stream alone; a large common offset of a row (mean far above the deviation) does not cost accuracy."""
     g = torch.Generator().manual_seed(W)
-    x, y = rnd(g, 5, W).float(), q16(rnd(g, 5, W) + 20)
+    for T in (5, 1030) if W <= 1024 else (5,):
+        sandwich(W, T, device, dtype, g)
+
+
+def sandwich(W, T, device, dtype, g):
+    x, y = rnd(g, T, W).float(), q16(rnd(g, T, W) + 20)
     wp, bp, add, w, b = (rnd(g, W).float() for _ in range(5))
     D = lambda t: None if t is None else t.to(device)      # noqa: E731
     sd = {"p": wp.double(), "p.b": bp.double(), "n": w.double(), "n.b": b.double()}
