@@ -81,11 +81,12 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(const T* __restrict__ u,
 // The same for taps <= 4 with 16-byte accesses: a thread owns EV adjacent channels and walks its `rows`
 // tokens with the three previous inputs in registers (weights right-aligned in a 4-tap window, the
 // unused leading taps zero), so every input row is read once per tile instead of once per tap.
-// Needs C % EV == 0 and 16-byte aligned rows of u, out and the state.
+// Needs C % EV == 0 and 16-byte aligned rows of u, out and the state.  new_state != null (steps of single tokens): the thread also
+// leaves its channels' last inputs there (the same tensor as `state`: it has read them before).
 template <typename T>
 __global__ __launch_bounds__(256) void conv_silu_vec_kernel(const T* __restrict__ u, long us, int C, int taps,
                                                             const float* __restrict__ w, const float* __restrict__ bias,
-                                                            const T* __restrict__ state, const int* __restrict__ cu,
+                                                            const T* state, T* new_state, const int* __restrict__ cu,
                                                             const int* __restrict__ slots,
                                                             const int* __restrict__ positions, T* __restrict__ out,
                                                             long os, int act, int rows) {
@@ -161,6 +162,13 @@ __global__ __launch_bounds__(256) void conv_silu_vec_kernel(const T* __restrict_
         win[2][e] = cur[x][e];
       }
       strow(out + (long)(row0 + i + x) * os + c0, r);
+    }
+  }
+  if (new_state) {
+#pragma unroll
+    for (int x = 0; x < 3; ++x) {   // win[x] is the input 3 - x - 1 tokens before the last one
+      const int si = taps - 4 + x;
+      if (si >= 0) strow(new_state + ((long)slot * (taps - 1) + si) * C + c0, win[x]);
     }
   }
 }
@@ -608,15 +616,18 @@ int lk_conv_silu(const void* u, long us, int C, int taps, const float* w, const 
     // tokens per workgroup (a kernel argument: tiles of 4 tokens were tried for steps of few, long sequences, where 16-token
     // tiles leave a chip of 256 CUs a handful of waves each, and measured slower: 79 us against 61 us at 4 x 1,024 x 2,048)
     const int rows = kConvRows;
+    const bool one = max_len == 1;
     dim3 gv(S, (max_len + rows - 1) / rows, cblocks);
     if (esz == 2)
-      conv_silu_vec_kernel<bf16_t><<<gv, 256, 0, st>>>((const bf16_t*)u, us, C, taps, w, bias, (const bf16_t*)state, cu,
-                                                       slots, positions, (bf16_t*)out, os, act, rows);
+      conv_silu_vec_kernel<bf16_t><<<gv, 256, 0, st>>>((const bf16_t*)u, us, C, taps, w, bias, (const bf16_t*)state,
+                                                       one && taps > 1 ? (bf16_t*)state : nullptr, cu, slots, positions, (bf16_t*)out, os,
+                                                       act, rows);
     else
-      conv_silu_vec_kernel<float><<<gv, 256, 0, st>>>((const float*)u, us, C, taps, w, bias, (const float*)state, cu, slots,
-                                                      positions, (float*)out, os, act, rows);
+      conv_silu_vec_kernel<float><<<gv, 256, 0, st>>>((const float*)u, us, C, taps, w, bias, (const float*)state,
+                                                      one && taps > 1 ? (float*)state : nullptr, cu, slots, positions, (float*)out, os, act,
+                                                      rows);
     LK_CHECK_LAUNCH();
-    if (taps > 1) {
+    if (taps > 1 && !one) {
       if (esz == 2) conv_state_kernel<bf16_t><<<g2, 256, 0, st>>>((const bf16_t*)u, us, C, taps, (bf16_t*)state, cu, slots, positions);
       else conv_state_kernel<float><<<g2, 256, 0, st>>>((const float*)u, us, C, taps, (float*)state, cu, slots, positions);
       LK_CHECK_LAUNCH();

@@ -131,21 +131,16 @@ __global__ __launch_bounds__(256) void stream_layernorm_kernel(float* __restrict
 }
 
 // A sublayer boundary of a stream normed in front and behind:  x <- x + LN(y) wp + bp [+ add],  out = LN(x) w + b, the row in registers
-// between the four reductions.  RW threads per output row (a workgroup for few rows, one wave -- no barrier at all -- once there are
-// rows enough to fill the chip), columns as in the kernel above.
+// between the four reductions.  One workgroup per output row, columns as in the kernel above.
 //   idx == null: x is updated in place;  idx != null: row idx[r] of x and y is read, nothing of x is written.
-template <typename TY, typename TO, int MAXI, int V, int RW>
+template <typename TY, typename TO, int MAXI, int V>
 __global__ __launch_bounds__(256) void stream_sandwich_kernel(float* __restrict__ x, const TY* __restrict__ y, long ys,
                                                               const float* __restrict__ wp, const float* __restrict__ bp,
                                                               const float* __restrict__ add, const float* __restrict__ w,
                                                               const float* __restrict__ b, float eps, const long* __restrict__ idx,
-                                                              TO* __restrict__ out, long os, int W, long rows) {
+                                                              TO* __restrict__ out, long os, int W) {
   __shared__ float red[4];
-  const int tid = threadIdx.x % RW;
-  const long orow = (long)blockIdx.x * (256 / RW) + threadIdx.x / RW;
-  if (RW < 256 && orow >= rows) return;   // (whole waves; no barrier in that form)
-  const long row = idx ? idx[orow] : orow;
-  auto row_sum = [&](float t) { return RW == 64 ? wave_sum(t) : block_sum<4>(t, red); };
+  const long orow = blockIdx.x, row = idx ? idx[orow] : orow;
   const int ng = W / V;   // column groups (W % V == 0)
   float v[MAXI][V], xr[MAXI][V];
   auto ldn = [](const auto* p, float (&f)[V]) {
@@ -169,18 +164,18 @@ __global__ __launch_bounds__(256) void stream_sandwich_kernel(float* __restrict_
     for (int i = 0; i < MAXI; ++i)
 #pragma unroll
       for (int e = 0; e < V; ++e) s += v[i][e];
-    const float mean = row_sum(s) / (float)W;
+    const float mean = block_sum<4>(s, red) / (float)W;
     float q = 0.f;
 #pragma unroll
     for (int i = 0; i < MAXI; ++i)
-      if (tid + RW * i < ng) {
+      if ((int)threadIdx.x + 256 * i < ng) {
 #pragma unroll
         for (int e = 0; e < V; ++e) {
           v[i][e] -= mean;
           q += v[i][e] * v[i][e];
         }
       }
-    const float inv = 1.f / sqrtf(row_sum(q) / (float)W + eps);
+    const float inv = 1.f / sqrtf(block_sum<4>(q, red) / (float)W + eps);
 #pragma unroll
     for (int i = 0; i < MAXI; ++i)
 #pragma unroll
@@ -188,10 +183,10 @@ __global__ __launch_bounds__(256) void stream_sandwich_kernel(float* __restrict_
   };
 #pragma unroll
   for (int i = 0; i < MAXI; ++i) {
-    const int c = (tid + RW * i) * V;
+    const int c = (threadIdx.x + 256 * i) * V;
 #pragma unroll
     for (int e = 0; e < V; ++e) v[i][e] = xr[i][e] = 0.f;
-    if (tid + RW * i < ng) {
+    if ((int)threadIdx.x + 256 * i < ng) {
       ldn(x + row * W + c, xr[i]);
       if (y) ldn(y + row * ys + c, v[i]);
     }
@@ -199,8 +194,8 @@ __global__ __launch_bounds__(256) void stream_sandwich_kernel(float* __restrict_
   if (y) norm();
 #pragma unroll
   for (int i = 0; i < MAXI; ++i) {
-    const int c = (tid + RW * i) * V;
-    if (tid + RW * i < ng) {
+    const int c = (threadIdx.x + 256 * i) * V;
+    if ((int)threadIdx.x + 256 * i < ng) {
       float ww[V], bb[V];
       if (y) {
         ldn(wp + c, ww);
@@ -224,8 +219,8 @@ __global__ __launch_bounds__(256) void stream_sandwich_kernel(float* __restrict_
   norm();
 #pragma unroll
   for (int i = 0; i < MAXI; ++i) {
-    const int c = (tid + RW * i) * V;
-    if (tid + RW * i < ng) {
+    const int c = (threadIdx.x + 256 * i) * V;
+    if ((int)threadIdx.x + 256 * i < ng) {
       float ww[V], bb[V], r[V];
       ldn(w + c, ww);
       ldn(b + c, bb);
@@ -308,15 +303,10 @@ int launch_sandwich(float* x, const void* y, long ys, const float* wp, const flo
                     float eps, const long* idx, void* out, long os, long rows, int W, hipStream_t st) {
   const auto a16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };   // (a null pointer passes)
   const bool vec = W % 4 == 0 && ys % 4 == 0 && os % 4 == 0 && a16(y) && a16(out) && a16(x) && a16(wp) && a16(bp) && a16(add) && a16(w) && a16(b);
-#define LK_SW_(MAXI, V, RW)                                                                                              \
-  stream_sandwich_kernel<TY, TO, MAXI, V, RW><<<(unsigned)((rows + 256 / RW - 1) / (256 / RW)), 256, 0, st>>>(           \
-      x, (const TY*)y, ys, wp, bp, add, w, b, eps, idx, (TO*)out, os, W, rows)
-#define LK_SW(MAXI, V) LK_SW_(MAXI, V, 256)
-  if (vec && rows >= 1024 && W <= 2048) {
-    if (W <= 512) LK_SW_(2, 4, 64);
-    else if (W <= 1024) LK_SW_(4, 4, 64);
-    else LK_SW_(8, 4, 64);
-  } else if (vec) {
+#define LK_SW(MAXI, V)                                                                                                       \
+  stream_sandwich_kernel<TY, TO, MAXI, V><<<(unsigned)rows, 256, 0, st>>>(x, (const TY*)y, ys, wp, bp, add, w, b, eps, idx, \
+                                                                          (TO*)out, os, W)
+  if (vec) {
     if (W <= 1024) LK_SW(1, 4);
     else if (W <= 2048) LK_SW(2, 4);
     else if (W <= 4096) LK_SW(4, 4);
@@ -329,7 +319,6 @@ int launch_sandwich(float* x, const void* y, long ys, const float* wp, const flo
     else return -1;
   }
 #undef LK_SW
-#undef LK_SW_
   LK_CHECK_LAUNCH();
   return 0;
 }

@@ -318,9 +318,6 @@ class KebepelModel(nn.Module):
         eps, dt, n = self.cfg.norm_eps, self.dtype, len(self.runs)
         x, _ = ops.embed_stream(ids, self.embed, dt)
         step = lambda t: None if t is None else self.steps[t]
-        idx = meta.logits_idx
-        if idx is None:
-            idx = torch.arange(x.shape[0], dtype=torch.long, device=x.device)
         h = ops.stream_sandwich_layernorm(x, None, None, None, step(self.runs[0][1]), *self.layers[self.runs[0][0]].ln("norm1"), eps, dt)
         for i, (li, _) in enumerate(self.runs):
             L = self.layers[li]
@@ -333,7 +330,8 @@ class KebepelModel(nn.Module):
                 ops.stream_sandwich_layernorm(t, y, *L.ln(post), None, self.final_norm, self.final_norm_b, eps, dt)
                 taps.append(t)
             if i + 1 == n:
-                return ops.stream_sandwich_layernorm(x, y, *L.ln(post), None, self.final_norm, self.final_norm_b, eps, dt, idx=idx)
+                return ops.stream_sandwich_layernorm(x, y, *L.ln(post), None, self.final_norm, self.final_norm_b, eps, dt,
+                                                     idx=meta.logits_idx)
             h = ops.stream_sandwich_layernorm(x, y, *L.ln(post), step(self.runs[i + 1][1]), *self.layers[self.runs[i + 1][0]].ln("norm1"), eps, dt)
 
     def head(self, hidden):
